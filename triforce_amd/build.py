@@ -1,38 +1,59 @@
-"""Build libtriforce_hip.so (gfx950) in-tree with hipcc.  No JIT cache: the .so travels with the tree."""
+"""Build the HIP libraries (gfx950) in-tree with hipcc.  No JIT cache: the .so files travel with the tree.
+
+Two libraries: ``core`` (libtriforce_hip.so: the Llama / TriForce kernels, sampling, collectives) and ``latent``
+(libtriforce_latent.so: the latent-attention family), so that a program which needs one of them compiles only that one."""
 import os
 import shutil
 import subprocess
+from concurrent.futures import ThreadPoolExecutor
 
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
+INCLUDE = os.path.abspath(os.path.join(HERE, "..", "include"))
 LIB_DIR = os.path.join(HERE, "lib")
 LIB_PATH = os.path.join(LIB_DIR, "libtriforce_hip.so")
+LATENT_LIB_PATH = os.path.join(LIB_DIR, "libtriforce_latent.so")
 SOURCES = ["attn.hip", "retrieval.hip", "elementwise.hip", "sampling.hip", "offload.hip", "gemv.hip", "allreduce.hip", "draft.hip", "draft_persist.hip", "topp_multi.hip", "abi.hip"]
+LIBRARIES = {
+    "core": (LIB_PATH, SOURCES, ["common.h", "tree_mask.h", "select_common.h"], ["triforce_hip.h"]),
+    "latent": (LATENT_LIB_PATH, ["latent_gemm.hip", "latent_attn.hip", "latent_ops.hip"], ["latent_common.h"],
+               ["triforce_latent.h"]),
+}
 # -amdgpu-kernarg-preload-count: the leading pointer / scalar kernel arguments (up to 14 dwords) arrive in SGPRs with the
 # dispatch instead of through s_load + s_waitcnt at the top of every kernel (gfx950 hardware feature; the compiler keeps a
 # backward-compatible entry for firmware without it).  The decode kernels order their arguments for it (csrc/gemv.hip).
+# -packed-fp32-ops: no v_pk_add / mul / fma_f32 out of ordinary float code (some of their forms are unreliable here).
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-shared", "-ffp-contract=off",
-         "-fno-gpu-rdc", "-Wno-unused-result", "-mllvm", "-amdgpu-kernarg-preload-count=14"]
+         "-fno-gpu-rdc", "-Wno-unused-result", "-mllvm", "-amdgpu-kernarg-preload-count=14",
+         "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def hipcc_path():
     p = shutil.which("hipcc") or "/opt/rocm/bin/hipcc"
     if not os.path.exists(p):
-        raise RuntimeError("hipcc not found: cannot build libtriforce_hip.so")
+        raise RuntimeError("hipcc not found: cannot build the HIP libraries")
     return p
 
 
-def sources():
-    return [os.path.join(CSRC, s) for s in SOURCES if os.path.exists(os.path.join(CSRC, s))]
+def sources(name="core"):
+    return [os.path.join(CSRC, s) for s in LIBRARIES[name][1]]
 
 
-def needs_build():
-    if not os.path.exists(LIB_PATH):
+def needs_build(name="core"):
+    """Is the library missing or older than something it is made from?"""
+    path, _, headers, public = LIBRARIES[name]
+    if not os.path.exists(path):
         return True
-    t = os.path.getmtime(LIB_PATH)
-    deps = sources() + [os.path.join(CSRC, "common.h"), os.path.join(CSRC, "tree_mask.h"), os.path.join(CSRC, "select_common.h"),
-                        os.path.join(HERE, "..", "include", "triforce_hip.h"), os.path.abspath(__file__)]   # (flags live here)
-    return any(os.path.getmtime(d) > t for d in deps if os.path.exists(d))
+    t = os.path.getmtime(path)
+    deps = sources(name) + [os.path.join(CSRC, h) for h in headers] + [os.path.join(INCLUDE, h) for h in public] \
+        + [os.path.abspath(__file__)]                                                                      # (flags live here)
+    return any(os.path.getmtime(d) > t for d in deps)
+
+
+def _run(cmd, verbose):
+    if verbose:
+        print("[triforce_amd.build]", " ".join(cmd), flush=True)
+    subprocess.run(cmd, check=True)
 
 
 def build_variant(name, defines, verbose=True):
@@ -43,24 +64,36 @@ def build_variant(name, defines, verbose=True):
     flags = [f for f in FLAGS if f not in drop]
     if "kernarg-preload" in drop:                                # "!kernarg-preload": build without the preload flag pair
         flags = [f for f in flags if f != "-mllvm" and not f.startswith("-amdgpu-kernarg-preload-count")]
-    cmd = [hipcc_path()] + flags + [d if d.startswith("-") else f"-D{d}" for d in defines if not d.startswith("!")] \
-        + sources() + ["-o", out]
-    if verbose:
-        print("[triforce_amd.build]", " ".join(cmd), flush=True)
-    subprocess.run(cmd, check=True)
+    _run([hipcc_path()] + flags + [d if d.startswith("-") else f"-D{d}" for d in defines if not d.startswith("!")]
+         + sources() + ["-o", out], verbose)
     return out
 
 
-def build_library(force=False, verbose=True):
-    if not force and not needs_build():
-        return LIB_PATH
-    os.makedirs(LIB_DIR, exist_ok=True)
-    cmd = [hipcc_path()] + FLAGS + sources() + ["-o", LIB_PATH]
-    if verbose:
-        print("[triforce_amd.build]", " ".join(cmd), flush=True)
-    subprocess.run(cmd, check=True)
-    return LIB_PATH
+def build_library(force=False, verbose=True, name="core", jobs=None):
+    """Compile one library (its files side by side) unless it is up to date; the finished file replaces the old one at once."""
+    path = LIBRARIES[name][0]
+    if not force and not needs_build(name):
+        return path
+    obj_dir = os.path.join(LIB_DIR, f"obj_{name}_{os.getpid()}")
+    os.makedirs(obj_dir, exist_ok=True)
+    try:
+        cc = hipcc_path()
+        pairs = [(s, os.path.join(obj_dir, os.path.basename(s) + ".o")) for s in sources(name)]
+        compile_flags = [f for f in FLAGS if f != "-shared"]
+        jobs = jobs or min(8, int(os.environ.get("MAX_JOBS", "8")), len(pairs))
+        with ThreadPoolExecutor(jobs) as pool:
+            list(pool.map(lambda so: _run([cc] + compile_flags + ["-c", so[0], "-o", so[1]], verbose), pairs))
+        tmp = path + f".{os.getpid()}"
+        _run([cc, "--offload-arch=gfx950", "-fPIC", "-shared", "-fno-gpu-rdc"] + [o for _, o in pairs] + ["-o", tmp], verbose)
+        os.replace(tmp, path)
+    finally:
+        shutil.rmtree(obj_dir, ignore_errors=True)
+    return path
+
+
+def build_all(force=False, verbose=True):
+    return [build_library(force=force, verbose=verbose, name=n) for n in LIBRARIES]
 
 
 if __name__ == "__main__":
-    build_library(force=True)
+    build_all(force=True)

@@ -1,0 +1,591 @@
+// Attention of the latent family for gfx950.
+//
+// Decode (attn_latent_kernel): the query has been taken through the key up-projection, so the cached row itself is the key
+// ([latent | rotated]) and its latent part the value, for every head: one KV stream shared by all heads.  A workgroup walks the
+// 64-key pages of its split; the page goes global -> registers -> LDS (the next page's loads are in flight while this one is
+// used).  Scores are computed transposed (S^T = K Q^T: rows keys, columns heads), so that a lane owns one head's statistics;
+// wave w takes keys 16w .. 16w+15.  The weights go to LDS as [head][key] and every wave then accumulates its share of the
+// latent columns, O^T = C^T P^T, with the transposed operand read straight from the key-major page (ds_read_b64_tr_b16).
+//
+// Prefill (attn_prefill_kernel): keys and values up-projected once per chunk, flash attention with 16 * QT query rows per wave,
+// four waves sharing the key / value tile.  Also transposed: the S^T result registers of two 16-key tiles ARE the P operand of
+// one PV product (the value operand is read with the matching key order), so the weights never leave the registers.
+#include "latent_common.h"
+
+#define NEG_INF (-__builtin_inff())
+#define LOG2E 1.4426950408889634f
+
+// ---------------------------------------------------------------------------------------------------------------- decode
+// Weights as two bfloat16 (value and remainder): the PV product then sees them to 16 bits like the fp32 softmax made them.
+template <typename T> struct DecodeCfg { static constexpr int PARTS = sizeof(T) == 2 ? 2 : 1; };
+
+// WC > 0: chunks (W / 32) at compile time with the register look-ahead; 0: any width up to the LDS limit.
+template <typename T, int NW, int HT, int NTW, int WC>
+__global__ __launch_bounds__(NW * 64, 1) void attn_latent_kernel(const T* __restrict__ q, const T* __restrict__ cache, int n_pages,
+                                                              const int32_t* __restrict__ table, int table_ld,
+                                                              const int32_t* __restrict__ len, T* __restrict__ out,
+                                                              float* __restrict__ ws, int H, int C, int R, float scale,
+                                                              int nsplit, int rows) {
+    typedef typename El<T>::Frag Frag;
+    constexpr int KT = 16 * NW, NT = NW * 64, EPV = 16 / sizeof(T), PADE = EPV;
+    constexpr int PARTS = DecodeCfg<T>::PARTS;
+    extern __shared__ __align__(16) char smem[];
+    [[maybe_unused]] const int wc = (C + R) >> 5;
+    const int W = C + R, ldk = (WC ? WC * 32 : W) + PADE, ldp = KT + PADE;
+    T* Kt = (T*)smem;                                         // [KT][ldk]
+    T* Qs = Kt + KT * ldk;                                    // [16 HT][ldk]
+    T* Ps = Qs + 16 * HT * ldk;                               // [PARTS][16 HT][ldp]
+    float* red = (float*)(Ps + PARTS * 16 * HT * ldp);        // [NW][16 HT]
+    const int split = blockIdx.x, h0 = blockIdx.y * 16 * HT, row = blockIdx.z;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g = lane >> 4, i = lane & 15;
+    const int n = len[row];
+    const int ntiles = n > 0 ? (n + KT - 1) / KT : 0;
+    const int per = (ntiles + nsplit - 1) / nsplit;
+    const int t_beg = min(split * per, ntiles), t_end = min(ntiles, t_beg + per);
+    const int ppr = (WC ? WC * 32 : W) / EPV;                 // 16-byte pieces per row
+    const int32_t* tab = table + (int64_t)row * table_ld;
+
+    for (int p = tid; p < 16 * HT * ppr; p += NT) {           // queries of this head group (heads past H: zeros)
+        const int r = p / ppr, c = p - r * ppr;
+        uint4 v = {0, 0, 0, 0};
+        if (h0 + r < H) v = *reinterpret_cast<const uint4*>(q + ((int64_t)row * H + h0 + r) * W + EPV * c);
+        *reinterpret_cast<uint4*>(Qs + r * ldk + EPV * c) = v;
+    }
+    constexpr int NPRE = WC ? (KT * WC * 32 / EPV) / NT : 1;  // pieces per thread and tile
+    uint4 pre[NPRE];
+    auto page_base = [&](int t) {
+        const int k0 = t * KT;
+        int pg = tab[k0 / TFL_PAGE];
+        pg = pg < 0 ? 0 : (pg >= n_pages ? n_pages - 1 : pg);
+        return (int64_t)pg * TFL_PAGE + (k0 & (TFL_PAGE - 1));
+    };
+    auto fetch = [&](int t) {
+        const T* base = cache + page_base(t) * W;
+#pragma unroll
+        for (int j = 0; j < NPRE; ++j)
+            pre[j] = *reinterpret_cast<const uint4*>(base + (int64_t)(tid + j * NT) * EPV);
+    };
+    f32x4 o[HT][NTW];
+    float m_run[HT], l_run[HT];
+#pragma unroll
+    for (int h = 0; h < HT; ++h) {
+        m_run[h] = NEG_INF;
+        l_run[h] = 0.f;
+#pragma unroll
+        for (int t = 0; t < NTW; ++t) o[h][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    if (WC && t_beg < t_end) fetch(t_beg);
+    for (int t = t_beg; t < t_end; ++t) {
+        const int k0 = t * KT;
+        if constexpr (WC > 0) {
+#pragma unroll
+            for (int j = 0; j < NPRE; ++j) {
+                const int p = tid + j * NT, r = p / ppr, c = p - r * ppr;
+                uint4 v = pre[j];
+                if (k0 + r >= n) v = uint4{0, 0, 0, 0};       // rows past the end: never let stale contents into 0 * x
+                *reinterpret_cast<uint4*>(Kt + r * ldk + EPV * c) = v;
+            }
+        } else {
+            const T* base = cache + page_base(t) * W;
+            for (int p = tid; p < KT * ppr; p += NT) {
+                const int r = p / ppr, c = p - r * ppr;
+                uint4 v = {0, 0, 0, 0};
+                if (k0 + r < n) v = *reinterpret_cast<const uint4*>(base + (int64_t)r * W + EPV * c);
+                *reinterpret_cast<uint4*>(Kt + r * ldk + EPV * c) = v;
+            }
+        }
+        __syncthreads();
+        if (WC && t + 1 < t_end) fetch(t + 1);
+        f32x4 s[HT];
+#pragma unroll
+        for (int h = 0; h < HT; ++h) s[h] = f32x4{0.f, 0.f, 0.f, 0.f};
+        const T* kp = Kt + (16 * wave + i) * ldk + 8 * g;
+        const T* qp = Qs + i * ldk + 8 * g;
+        auto chunk = [&](int c) {
+            const Frag a = load_frag(kp + 32 * c);
+#pragma unroll
+            for (int h = 0; h < HT; ++h) s[h] = El<T>::mma(a, load_frag(qp + h * 16 * ldk + 32 * c), s[h]);
+        };
+        if constexpr (WC > 0) {
+#pragma unroll 6
+            for (int c = 0; c < WC; ++c) chunk(c);
+        } else {
+            for (int c = 0; c < wc; ++c) chunk(c);
+        }
+#pragma unroll
+        for (int h = 0; h < HT; ++h) {
+            float mx = NEG_INF;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                s[h][r] = k0 + 16 * wave + 4 * g + r < n ? s[h][r] * scale : NEG_INF;
+                mx = fmaxf(mx, s[h][r]);
+            }
+            mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+            mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+            if (g == 0) red[wave * 16 * HT + 16 * h + i] = mx;
+        }
+        __syncthreads();
+        float alpha[HT];
+#pragma unroll
+        for (int h = 0; h < HT; ++h) {
+            float mx = m_run[h];
+#pragma unroll
+            for (int w = 0; w < NW; ++w) mx = fmaxf(mx, red[w * 16 * HT + 16 * h + i]);
+            alpha[h] = exp2f((m_run[h] - mx) * LOG2E);        // (the tile's first key is visible: mx is finite)
+            m_run[h] = mx;
+            f32x4 p, lo;
+            float sum = 0.f;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                p[r] = exp2f((s[h][r] - mx) * LOG2E);
+                sum += p[r];
+                lo[r] = p[r] - (float)(T)p[r];
+            }
+            l_run[h] = l_run[h] * alpha[h] + sum;
+            T* dst = Ps + (16 * h + i) * ldp + 16 * wave + 4 * g;
+            store_quad(dst, p);
+            if constexpr (PARTS == 2) store_quad(dst + 16 * HT * ldp, lo);
+        }
+        __syncthreads();
+#pragma unroll
+        for (int h = 0; h < HT; ++h)
+#pragma unroll
+            for (int x = 0; x < NTW; ++x)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) o[h][x][r] *= alpha[h];
+#pragma unroll
+        for (int c = 0; c < KT / 32; ++c) {
+            Frag b[HT][PARTS];
+#pragma unroll
+            for (int h = 0; h < HT; ++h)
+#pragma unroll
+                for (int z = 0; z < PARTS; ++z) b[h][z] = load_frag(Ps + (z * 16 * HT + 16 * h + i) * ldp + 32 * c + 8 * g);
+#pragma unroll
+            for (int x = 0; x < NTW; ++x) {
+                const int col = 16 * (wave * NTW + x);
+                if (col < C) {
+                    const Frag a = load_frag_t(Kt, ldk, 32 * c + 8 * g, 32 * c + 8 * g + 4, col, i);
+#pragma unroll
+                    for (int h = 0; h < HT; ++h)
+#pragma unroll
+                        for (int z = 0; z < PARTS; ++z) o[h][x] = El<T>::mma(a, b[h][z], o[h][x]);
+                }
+            }
+        }
+        __syncthreads();
+    }
+    // sum of the weights: lane groups hold different keys, waves too
+#pragma unroll
+    for (int h = 0; h < HT; ++h) {
+        float l = l_run[h];
+        l += __shfl_xor(l, 16, 64);
+        l += __shfl_xor(l, 32, 64);
+        if (g == 0) red[wave * 16 * HT + 16 * h + i] = l;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int h = 0; h < HT; ++h) {
+        const int head = h0 + 16 * h + i;
+        if (head >= H) continue;
+        float l = 0.f;
+#pragma unroll
+        for (int w = 0; w < NW; ++w) l += red[w * 16 * HT + 16 * h + i];
+        if (nsplit == 1) {
+            const float inv = l > 0.f ? 1.0f / l : 0.f;
+#pragma unroll
+            for (int x = 0; x < NTW; ++x) {
+                const int col = 16 * (wave * NTW + x) + 4 * g;
+                if (col < C) {
+                    f32x4 v = o[h][x];
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) v[r] *= inv;
+                    store_quad(out + ((int64_t)row * H + head) * C + col, v);
+                }
+            }
+        } else {
+            const int64_t at = ((int64_t)row * H + head) * nsplit + split;
+            float* wo = ws + at * C;
+#pragma unroll
+            for (int x = 0; x < NTW; ++x) {
+                const int col = 16 * (wave * NTW + x) + 4 * g;
+                if (col < C && l > 0.f) *reinterpret_cast<f32x4*>(wo + col) = o[h][x];   // (empty splits are not read either)
+            }
+            if (wave == 0 && g == 0) {
+                float* ml = ws + (int64_t)rows * H * nsplit * C + at * 2;
+                ml[0] = m_run[h];
+                ml[1] = l;
+            }
+        }
+    }
+}
+
+// Merge of the splits: one workgroup per (head, row).
+template <typename T>
+__global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restrict__ ws, T* __restrict__ out, int rows, int H,
+                                                           int C, int nsplit) {
+    __shared__ float wgt[256];
+    __shared__ f32x4 acc[256];
+    const int head = blockIdx.x, row = blockIdx.y, tid = threadIdx.x;
+    const int64_t at = ((int64_t)row * H + head) * nsplit;
+    const float* ml = ws + (int64_t)rows * H * nsplit * C + at * 2;
+    // thread s owns split s (nsplit <= 256); an empty split has weight 0 and its partial row is never read
+    __shared__ float red[8];
+    const float ls = tid < nsplit ? ml[2 * tid + 1] : 0.f;
+    const float ms = ls > 0.f ? ml[2 * tid] : NEG_INF;
+    float m = ms;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) m = fmaxf(m, __shfl_xor(m, o, 64));
+    if ((tid & 63) == 0) red[4 + (tid >> 6)] = m;
+    __syncthreads();
+    m = fmaxf(fmaxf(red[4], red[5]), fmaxf(red[6], red[7]));
+    const float w = ls > 0.f ? exp2f((ms - m) * LOG2E) : 0.f;
+    const float l = block_sum256(w * ls, red);
+    wgt[tid] = l > 0.f ? w / l : 0.f;
+    __syncthreads();
+    const int nq = C >> 2, lanes = nq < 256 ? nq : 256, grps = 256 / lanes;      // groups of threads share the splits
+    const int gi = tid / lanes, li = tid - gi * lanes;
+    for (int q0 = 0; q0 < nq; q0 += lanes) {
+        const int q = q0 + li;
+        f32x4 v = {0.f, 0.f, 0.f, 0.f};
+        if (gi < grps && q < nq)
+            for (int s = gi; s < nsplit; s += grps)
+                if (wgt[s] > 0.f) {
+                    const f32x4 z = *reinterpret_cast<const f32x4*>(ws + (at + s) * C + 4 * q);
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) v[r] = fmaf(z[r], wgt[s], v[r]);
+                }
+        acc[tid] = v;
+        __syncthreads();
+        if (gi == 0 && q < nq) {
+            for (int k = 1; k < grps; ++k) {
+                const f32x4 z = acc[k * lanes + li];
+#pragma unroll
+                for (int r = 0; r < 4; ++r) v[r] += z[r];
+            }
+            store_quad(out + ((int64_t)row * H + head) * C + 4 * q, v);
+        }
+        __syncthreads();
+    }
+}
+
+#define TFL_MAX_SPLIT 256
+
+extern "C" int64_t tfl_attn_decode_ws_floats(int rows, int H, int C, int nsplit) {
+    if (rows < 1 || H < 1 || C < 1 || nsplit < 1) return 0;
+    return nsplit == 1 ? 0 : (int64_t)rows * H * nsplit * (C + 2);
+}
+
+// One workgroup per CU (256) as long as a split keeps at least two pages of keys.
+extern "C" int tfl_attn_decode_pick_nsplit(int rows, int H, int max_len) {
+    if (rows < 1 || H < 1 || max_len < 1) return 1;
+    const int groups = H <= 16 ? 1 : (H + 31) / 32;
+    int n = 256 / (rows * groups);
+    const int cap = (max_len + 2 * TFL_PAGE - 1) / (2 * TFL_PAGE);
+    if (n > cap) n = cap;
+    if (n > TFL_MAX_SPLIT) n = TFL_MAX_SPLIT;
+    return n < 1 ? 1 : n;
+}
+
+template <typename T, int NW, int HT, int NTW, int WC>
+static int launch_latent(const void* q, const void* cache, int n_pages, const int32_t* table, int table_ld, const int32_t* len,
+                         void* out, float* ws, int rows, int H, int C, int R, float scale, int nsplit, hipStream_t st) {
+    const int W = C + R, pad = 16 / (int)sizeof(T), KT = 16 * NW;
+    const size_t lds = sizeof(T) * ((size_t)(KT + 16 * HT) * (W + pad) + (size_t)DecodeCfg<T>::PARTS * 16 * HT * (KT + pad))
+                     + sizeof(float) * NW * 16 * HT;
+    if (lds > 160 * 1024) return TF_ERANGE;
+    auto k = attn_latent_kernel<T, NW, HT, NTW, WC>;
+    static bool attr = false;
+    if (!attr) {
+        const hipError_t e = hipFuncSetAttribute((const void*)k, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+        if (e != hipSuccess) return (int)e;
+        attr = true;
+    }
+    hipLaunchKernelGGL(k, dim3(nsplit, (H + 16 * HT - 1) / (16 * HT), rows), dim3(NW * 64), lds, st, (const T*)q, (const T*)cache,
+                       n_pages, table, table_ld, len, (T*)out, ws, H, C, R, scale, nsplit, rows);
+    TFL_LAUNCH_CHECK();
+    if (nsplit > 1) {
+        hipLaunchKernelGGL((latent_merge_kernel<T>), dim3(H, rows), dim3(256), 0, st, ws, (T*)out, rows, H, C, nsplit);
+        TFL_LAUNCH_CHECK();
+    }
+    return TF_OK;
+}
+
+extern "C" int tfl_attn_decode(const void* q, const void* cache, int n_pages, const int32_t* table, int table_ld, const int32_t* len,
+                               void* out, float* ws, int64_t ws_floats, int rows, int H, int C, int R, float scale, int nsplit,
+                               int dtype, void* stream) {
+    if (!q || !cache || !table || !len || !out || rows < 1 || rows > 65535 || H < 1 || n_pages < 1 || table_ld < 1) return TF_EINVAL;
+    if (C < 32 || (C & 31) || R < 0 || (R & 31) || nsplit < 1 || nsplit > TFL_MAX_SPLIT) return TF_EINVAL;
+    if (nsplit > 1 && (!ws || ws_floats < tfl_attn_decode_ws_floats(rows, H, C, nsplit))) return TF_ENOSPC;
+    hipStream_t st = (hipStream_t)stream;
+#define GO(T, NW, HT, NTW, WC) \
+    return launch_latent<T, NW, HT, NTW, WC>(q, cache, n_pages, table, table_ld, len, out, ws, rows, H, C, R, scale, nsplit, st)
+    if (dtype == 0) {
+        if (C == 512 && R == 64) { if (H <= 16) GO(bf16, 4, 1, 8, 18); GO(bf16, 4, 2, 8, 18); }
+        if (C <= 128) { if (H <= 16) GO(bf16, 4, 1, 2, 0); GO(bf16, 4, 2, 2, 0); }
+        if (C <= 512) { if (H <= 16) GO(bf16, 4, 1, 8, 0); GO(bf16, 4, 2, 8, 0); }
+        if (C <= 1024) GO(bf16, 2, 1, 32, 0);
+        return TF_ERANGE;
+    }
+    if (dtype == 1) {
+        if (C <= 128) { if (H <= 16) GO(float, 4, 1, 2, 0); GO(float, 4, 2, 2, 0); }
+        if (C <= 512) GO(float, 2, 1, 16, 0);
+        return TF_ERANGE;
+    }
+#undef GO
+    return TF_EINVAL;
+}
+
+// --------------------------------------------------------------------------------------------------------------- prefill
+// KT keys per tile, QT 16-row query tiles per wave, up to DK 32-wide chunks of query-key size (NC unrotated ones first) and DV
+// 16-wide tiles of value size.  EXACT: the sizes are exactly NCX, DK, DV (no bounds in the inner loops, register look-ahead).
+template <typename T, int KT, int QT, int DK, int DV, int NCX>
+__global__ __launch_bounds__(256, 1) void attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ kv, const T* __restrict__ ck,
+                                                           const int32_t* __restrict__ seq, const int32_t* __restrict__ pos,
+                                                           const float* __restrict__ cosb, const float* __restrict__ sinb,
+                                                           int half, int max_pos, const T* __restrict__ gate, int64_t ld_gate,
+                                                           T* __restrict__ out, int64_t ld_out, int tq, int tk, int H, int N, int R,
+                                                           int V, int C, float scale) {
+    typedef typename El<T>::Frag Frag;
+    constexpr bool EXACT = NCX > 0;
+    constexpr int EPV = 16 / sizeof(T), PADE = EPV, QB = 64 * QT;
+    extern __shared__ __align__(16) char smem[];
+    const int nc = EXACT ? NCX : N >> 5, dk = EXACT ? DK : (N + R) >> 5, dv = EXACT ? DV : V >> 4;
+    const int D = 32 * dk, ldk = D + PADE, ldv = 16 * dv + PADE;
+    T* Ks = (T*)smem;                                         // [KT][ldk]
+    T* Vs = Ks + KT * ldk;                                    // [KT][ldv]
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g = lane >> 4, i = lane & 15;
+    const int h = blockIdx.y;
+    const int32_t* sq = seq + 4 * blockIdx.z;
+    const int q_at = sq[0], nq = sq[1], k_at = sq[2], nk = sq[3];
+    const int qb = (gridDim.x - 1 - blockIdx.x) * QB;         // longest blocks first
+    if (qb >= nq || nq < 1 || nk < nq || q_at < 0 || k_at < 0 || q_at + nq > tq || k_at + nk > tk) return;
+    const int past = nk - nq;
+    const int64_t ld_kv = (int64_t)H * (N + V), ld_ck = C + R;
+
+    Frag qf[QT][DK];
+    int qpos[QT];                                             // key index of the lane's own query token
+#pragma unroll
+    for (int t = 0; t < QT; ++t) {
+        const int j = qb + 16 * (wave * QT + t) + i;
+        qpos[t] = past + j;
+        const int64_t tok = q_at + min(j, nq - 1);
+        const T* src = q + (tok * H + h) * (int64_t)(N + R) + 8 * g;
+        int p = pos[tok];
+        p = p < 0 ? 0 : (p >= max_pos ? max_pos - 1 : p);
+#pragma unroll
+        for (int c = 0; c < DK; ++c) {
+            if (!EXACT && c >= dk) { qf[t][c] = Frag{}; continue; }
+            Frag f = load_frag(src + 32 * c);
+            if (c >= nc) {
+                const int pr = (c - nc) * 16 + 4 * g;
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (pr + e < half) {
+                        const float cs = cosb[(int64_t)p * half + pr + e], sn = sinb[(int64_t)p * half + pr + e];
+                        const float u = (float)f[2 * e], v = (float)f[2 * e + 1];
+                        f[2 * e] = (T)(u * cs - v * sn);
+                        f[2 * e + 1] = (T)(v * cs + u * sn);
+                    }
+            }
+            qf[t][c] = f;
+        }
+    }
+    f32x4 o[QT][DV];
+    float m_run[QT], l_run[QT];
+#pragma unroll
+    for (int t = 0; t < QT; ++t) {
+        m_run[t] = NEG_INF;
+        l_run[t] = 0.f;
+#pragma unroll
+        for (int d = 0; d < DV; ++d) o[t][d] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    const int last_q = min(qb + QB, nq) - 1;                  // last query row of the workgroup
+    const int ntiles = (past + last_q) / KT + 1;
+    const int first_qpos = past + qb + 16 * wave * QT;        // the wave's first row: tiles that end before it need no mask
+    const int kn = N / EPV, kr = R / EPV, vn = V / EPV, ppr = kn + kr + vn;   // 16-byte pieces per key
+    constexpr int NPRE = EXACT ? (KT * (32 * DK + 16 * DV) / EPV) / 256 : 1;
+    uint4 pre[NPRE];
+    auto piece = [&](int p, int t, bool zero, int& key, int& dst_v, int& dst_c) {
+        key = p / ppr;
+        int c = p - key * ppr;
+        const int64_t kk = k_at + min(t * KT + key, nk - 1);
+        const T* src;
+        if (c < kn) { src = kv + kk * ld_kv + (int64_t)h * N + EPV * c; dst_v = 0; dst_c = EPV * c; }
+        else if (c < kn + kr) { c -= kn; src = ck + kk * ld_ck + C + EPV * c; dst_v = 0; dst_c = N + EPV * c; }
+        else { c -= kn + kr; src = kv + kk * ld_kv + (int64_t)H * N + (int64_t)h * V + EPV * c; dst_v = 1; dst_c = EPV * c; }
+        uint4 v = {0, 0, 0, 0};
+        if (!zero) v = *reinterpret_cast<const uint4*>(src);
+        return v;
+    };
+    auto put = [&](int key, int dst_v, int dst_c, uint4 v) {
+        *reinterpret_cast<uint4*>(dst_v ? Vs + key * ldv + dst_c : Ks + key * ldk + dst_c) = v;
+    };
+    if constexpr (EXACT) {
+#pragma unroll
+        for (int j = 0; j < NPRE; ++j) {
+            int a, b, c;
+            pre[j] = piece(tid + 256 * j, 0, false, a, b, c);
+        }
+    }
+    for (int t = 0; t < ntiles; ++t) {
+        const int k0 = t * KT;
+        if constexpr (EXACT) {
+#pragma unroll
+            for (int j = 0; j < NPRE; ++j) {
+                int a, b, c;
+                (void)piece(tid + 256 * j, t, true, a, b, c);
+                put(a, b, c, pre[j]);
+            }
+        } else {
+            for (int p = tid; p < KT * ppr; p += 256) {
+                int a, b, c;
+                const uint4 v = piece(p, t, false, a, b, c);
+                put(a, b, c, v);
+            }
+        }
+        __syncthreads();
+        if constexpr (EXACT) {
+            if (t + 1 < ntiles) {
+#pragma unroll
+                for (int j = 0; j < NPRE; ++j) {
+                    int a, b, c;
+                    pre[j] = piece(tid + 256 * j, t + 1, false, a, b, c);
+                }
+            }
+        }
+        f32x4 s[KT / 16][QT];
+#pragma unroll
+        for (int kt = 0; kt < KT / 16; ++kt) {
+#pragma unroll
+            for (int u = 0; u < QT; ++u) s[kt][u] = f32x4{0.f, 0.f, 0.f, 0.f};
+            const T* kp = Ks + (16 * kt + i) * ldk + 8 * g;
+#pragma unroll
+            for (int c = 0; c < DK; ++c) {
+                if (EXACT || c < dk) {
+                    const Frag a = load_frag(kp + 32 * c);
+#pragma unroll
+                    for (int u = 0; u < QT; ++u) s[kt][u] = El<T>::mma(a, qf[u][c], s[kt][u]);
+                }
+            }
+        }
+        if (k0 + KT - 1 > first_qpos) {
+#pragma unroll
+            for (int kt = 0; kt < KT / 16; ++kt)
+#pragma unroll
+                for (int u = 0; u < QT; ++u)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r)
+                        if (k0 + 16 * kt + 4 * g + r > qpos[u]) s[kt][u][r] = NEG_INF;
+        }
+        Frag pf[QT][KT / 32];
+#pragma unroll
+        for (int u = 0; u < QT; ++u) {
+            float mx = NEG_INF;
+#pragma unroll
+            for (int kt = 0; kt < KT / 16; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[kt][u][r]);
+            mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+            mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+            mx = fmaxf(m_run[u], mx * scale);                 // (scale > 0; key 0 is visible to every row: finite from tile 0 on)
+            const float alpha = exp2f((m_run[u] - mx) * LOG2E), sc = scale * LOG2E, mb = mx * LOG2E;
+            m_run[u] = mx;
+            float sum = 0.f;
+#pragma unroll
+            for (int kt = 0; kt < KT / 16; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const float p = exp2f(fmaf(s[kt][u][r], sc, -mb));
+                    sum += p;
+                    pf[u][kt >> 1][(kt & 1) * 4 + r] = (T)p;
+                }
+            l_run[u] = l_run[u] * alpha + sum;
+#pragma unroll
+            for (int d = 0; d < DV; ++d)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) o[u][d][r] *= alpha;
+        }
+#pragma unroll
+        for (int d = 0; d < DV; ++d) {
+            if (EXACT || d < dv) {
+#pragma unroll
+                for (int c = 0; c < KT / 32; ++c) {
+                    const Frag a = load_frag_t(Vs, ldv, 32 * c + 4 * g, 32 * c + 16 + 4 * g, 16 * d, i);
+#pragma unroll
+                    for (int u = 0; u < QT; ++u) o[u][d] = El<T>::mma(a, pf[u][c], o[u][d]);
+                }
+            }
+        }
+        __syncthreads();
+    }
+#pragma unroll
+    for (int u = 0; u < QT; ++u) {
+        const int j = qb + 16 * (wave * QT + u) + i;
+        float l = l_run[u];
+        l += __shfl_xor(l, 16, 64);
+        l += __shfl_xor(l, 32, 64);
+        if (j >= nq) continue;
+        const float inv = 1.0f / l;
+        const int64_t tok = q_at + j;
+#pragma unroll
+        for (int d = 0; d < DV; ++d) {
+            if (!EXACT && d >= dv) continue;
+            const int col = h * V + 16 * d + 4 * g;
+            const f32x4 z = load_quad(gate + tok * ld_gate + col);
+            f32x4 v = o[u][d];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v[r] *= inv * sigmoid(z[r]);
+            store_quad(out + tok * ld_out + col, v);
+        }
+    }
+}
+
+template <typename T, int KT, int QT, int DK, int DV, int NCX>
+static int launch_prefill(const void* q, const void* kv, const void* ck, const int32_t* seq, int nseq, int max_new, const int32_t* pos,
+                          const float* cosb, const float* sinb, int half, int max_pos, const void* gate, int64_t ld_gate, void* out,
+                          int64_t ld_out, int tq, int tk, int H, int N, int R, int V, int C, float scale, hipStream_t st) {
+    const int pad = 16 / (int)sizeof(T);
+    const size_t lds = sizeof(T) * KT * (size_t)(N + R + V + 2 * pad);
+    if (lds > 160 * 1024) return TF_ERANGE;
+    auto k = attn_prefill_kernel<T, KT, QT, DK, DV, NCX>;
+    static bool attr = false;
+    if (!attr) {
+        const hipError_t e = hipFuncSetAttribute((const void*)k, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+        if (e != hipSuccess) return (int)e;
+        attr = true;
+    }
+    hipLaunchKernelGGL(k, dim3((max_new + 64 * QT - 1) / (64 * QT), H, nseq), dim3(256), lds, st, (const T*)q, (const T*)kv, (const T*)ck,
+                       seq, pos, cosb, sinb, half, max_pos, (const T*)gate, ld_gate, (T*)out, ld_out, tq, tk, H, N, R, V, C, scale);
+    TFL_LAUNCH_CHECK();
+    return TF_OK;
+}
+
+extern "C" int tfl_attn_prefill(const void* q, const void* kv, const void* ck, const int32_t* seq, int nseq, int max_new,
+                                const int32_t* pos, const float* cosb, const float* sinb, int half, int max_pos, const void* gate,
+                                int64_t ld_gate, void* out, int64_t ld_out, int tq, int tk, int H, int N, int R, int V, int C,
+                                float scale, int dtype, void* stream) {
+    if (!q || !kv || !ck || !seq || !pos || !gate || !out || nseq < 1 || nseq > 65535 || max_new < 1 || tq < 1 || tk < 1) return TF_EINVAL;
+    if (H < 1 || H > 65535 || N < 32 || (N & 31) || R < 0 || (R & 31) || V < 32 || (V & 31) || C < 32 || (C & 31)) return TF_EINVAL;
+    if (half < 0 || 2 * half > R || max_pos < 1 || (half && (!cosb || !sinb)) || !(scale > 0.f)) return TF_EINVAL;
+    if ((ld_gate & 3) || (ld_out & 3) || ld_gate < (int64_t)H * V || ld_out < (int64_t)H * V) return TF_EINVAL;
+    hipStream_t st = (hipStream_t)stream;
+#define GO(T, KT, QT, DK, DV, NCX)                                                                                               \
+    return launch_prefill<T, KT, QT, DK, DV, NCX>(q, kv, ck, seq, nseq, max_new, pos, cosb, sinb, half, max_pos, gate, ld_gate, \
+                                                  out, ld_out, tq, tk, H, N, R, V, C, scale, st)
+    const int D = N + R;
+    if (dtype == 0) {
+        if (N == 128 && R == 64 && V == 128) GO(bf16, 64, 2, 6, 8, 4);
+        if (D <= 96 && V <= 64) GO(bf16, 64, 1, 3, 4, 0);
+        if (D <= 192 && V <= 128) GO(bf16, 64, 1, 6, 8, 0);
+        if (D <= 384 && V <= 256) GO(bf16, 64, 1, 12, 16, 0);
+        return TF_ERANGE;
+    }
+    if (dtype == 1) {
+        if (D <= 96 && V <= 64) GO(float, 32, 1, 3, 4, 0);
+        if (D <= 192 && V <= 128) GO(float, 32, 1, 6, 8, 0);
+        if (D <= 384 && V <= 256) GO(float, 32, 1, 12, 16, 0);
+        return TF_ERANGE;
+    }
+#undef GO
+    return TF_EINVAL;
+}

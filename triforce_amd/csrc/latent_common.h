@@ -1,0 +1,132 @@
+// Element types and MFMA fragments shared by the latent-attention kernels (csrc/latent_*.hip).
+//
+// Every kernel is written once and instantiated for bfloat16 and for float.  A fragment is 8 elements of one matrix row: lane
+// (g = lane / 16, i = lane % 16) holds row i, k = 8g .. 8g+7 of a 16x32 tile.  bfloat16 feeds it to one 16x16x32 MFMA; float to
+// eight 16x16x4 MFMAs, the j-th taking element j of every lane (a permutation of the contraction index that both operands
+// share).  Result layout of both: lane (g, i) holds rows 4g .. 4g+3 of column i.
+#pragma once
+#include <hip/hip_runtime.h>
+#include <stdint.h>
+#include "../../include/triforce_latent.h"
+
+typedef __bf16 bf16;
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
+typedef float f32x8 __attribute__((ext_vector_type(8)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+template <typename T> struct El;
+template <> struct El<bf16> {
+    typedef bf16x8 Frag;
+    typedef bf16x4 Quad;
+    static __device__ __forceinline__ f32x4 mma(Frag a, Frag b, f32x4 c) {
+        return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+    }
+};
+template <> struct El<float> {
+    typedef f32x8 Frag;
+    typedef f32x4 Quad;
+    static __device__ __forceinline__ f32x4 mma(Frag a, Frag b, f32x4 c) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], b[j], c, 0, 0, 0);
+        return c;
+    }
+};
+
+template <typename T> __device__ __forceinline__ typename El<T>::Frag load_frag(const T* p) {
+    return *reinterpret_cast<const typename El<T>::Frag*>(p);
+}
+template <typename T> __device__ __forceinline__ typename El<T>::Frag load_frag_stream(const T* p) {
+    return __builtin_nontemporal_load(reinterpret_cast<const typename El<T>::Frag*>(p));
+}
+template <typename T> __device__ __forceinline__ void store_quad(T* p, f32x4 v) {
+    typename El<T>::Quad q;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) q[r] = (T)v[r];
+    *reinterpret_cast<typename El<T>::Quad*>(p) = q;
+}
+template <typename T> __device__ __forceinline__ f32x4 load_quad(const T* p) {
+    const typename El<T>::Quad q = *reinterpret_cast<const typename El<T>::Quad*>(p);
+    f32x4 v;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v[r] = (float)q[r];
+    return v;
+}
+
+// Transposed fragment from an LDS tile that is stored key-major ([key][column], row stride ld): lane (g, i) gets column
+// col + i of keys k0 .. k0+3 (elements 0-3) and k1 .. k1+3 (elements 4-7), where k0 / k1 are the lane's own (per g) key rows.
+// bfloat16: ds_read_b64_tr_b16 - the 16 lanes of a group address a 4 x 16 block (4 elements each) and get its columns back.
+__device__ __forceinline__ bf16x8 load_frag_t(const bf16* tile, int ld, int k0, int k1, int col, int i) {
+    typedef __attribute__((address_space(3))) bf16x4* lds4;
+    const bf16* p0 = tile + (k0 + (i >> 2)) * ld + col + 4 * (i & 3);
+    const bf16* p1 = tile + (k1 + (i >> 2)) * ld + col + 4 * (i & 3);
+    const bf16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds4)p0);
+    const bf16x4 b = __builtin_amdgcn_ds_read_tr16_b64_v4bf16((lds4)p1);
+    return __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7);
+}
+__device__ __forceinline__ f32x8 load_frag_t(const float* tile, int ld, int k0, int k1, int col, int i) {
+    f32x8 f;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        f[j] = tile[(k0 + j) * ld + col + i];
+        f[4 + j] = tile[(k1 + j) * ld + col + i];
+    }
+    return f;
+}
+
+// The tanh form of gelu: 0.5 z (1 + tanh(u)) = z / (1 + exp(-2u)), u = sqrt(2/pi) (z + 0.044715 z^3).
+__device__ __forceinline__ float gelu_tanh(float z) {
+    const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
+    return z / (1.0f + expf(-2.0f * u));
+}
+__device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+__device__ __forceinline__ float wave_sum64(float v) {
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
+    return v;
+}
+// Sum over a 256-thread workgroup; red = 4 floats of LDS, free again after the call's second barrier.
+__device__ __forceinline__ float block_sum256(float v, float* red) {
+    v = wave_sum64(v);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    v = red[0] + red[1] + red[2] + red[3];
+    __syncthreads();
+    return v;
+}
+
+// One cache row from raw latent / key values: latent / rms(latent) * w, rotated key.  One 256-thread workgroup.
+// src(c) reads raw element c of [latent C][key R].
+template <typename T, typename Src>
+__device__ __forceinline__ void cache_row_256(Src src, int C, int c_real, int R, const float* w, float eps, const float* cosr,
+                                              const float* sinr, int half, T* dst0, T* dst1, float* red) {
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < C; c += 256) {
+        const float f = src(c);
+        ss = fmaf(f, f, ss);
+    }
+    ss = block_sum256(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)c_real + eps);
+    for (int c = threadIdx.x; c < C; c += 256) {
+        const T o = (T)(src(c) * inv * w[c]);
+        if (dst0) dst0[c] = o;
+        if (dst1) dst1[c] = o;
+    }
+    for (int p = threadIdx.x; p < R / 2; p += 256) {
+        float u = src(C + 2 * p), v = src(C + 2 * p + 1);
+        if (p < half) {
+            const float cs = cosr[p], sn = sinr[p], a = u * cs - v * sn;
+            v = v * cs + u * sn;
+            u = a;
+        }
+        if (dst0) { dst0[C + 2 * p] = (T)u; dst0[C + 2 * p + 1] = (T)v; }
+        if (dst1) { dst1[C + 2 * p] = (T)u; dst1[C + 2 * p + 1] = (T)v; }
+    }
+}
+
+#define TFL_LAUNCH_CHECK()                      \
+    do {                                        \
+        hipError_t e__ = hipGetLastError();     \
+        if (e__ != hipSuccess) return (int)e__; \
+    } while (0)

@@ -1,0 +1,232 @@
+// Row kernels of the latent-attention family: residual / norm steps between layers, the prefill half of the input projection
+// (norms, rotation, cache append, gelu), the per-layer token gate, cache-row gather, and the set-up of a decode step.
+#include "latent_common.h"
+
+extern "C" int tfl_abi_version(void) { return 1; }
+
+template <typename T, typename Y>
+__global__ __launch_bounds__(256) void finish_kernel(const T* __restrict__ embed, const int64_t* __restrict__ ids, int vocab,
+                                                     const Y* __restrict__ y, int64_t ld_y, const float* __restrict__ y_w,
+                                                     const float* __restrict__ step, const float* __restrict__ norm_w,
+                                                     float* __restrict__ x, T* __restrict__ h, int width, int width_real,
+                                                     float eps) {
+    __shared__ float red[4];
+    const int row = blockIdx.x, nq = width >> 2;             // elements in groups of 4
+    float* xr = x + (int64_t)row * width;
+    const T* er = nullptr;
+    if (embed) {
+        int64_t id = ids[row];
+        id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+        er = embed + id * (int64_t)width;
+    }
+    const Y* yr = y ? y + (int64_t)row * ld_y : nullptr;
+    float yi = 0.f;
+    if (yr) {
+        float s = 0.f;
+        for (int q = threadIdx.x; q < nq; q += 256) {
+            const f32x4 v = load_quad(yr + 4 * q);
+            s += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+        }
+        s = block_sum256(s, red);
+        yi = 1.0f / sqrtf(s / (float)width_real + eps);
+    }
+    float s = 0.f;
+    for (int q = threadIdx.x; q < nq; q += 256) {
+        f32x4 v = er ? load_quad(er + 4 * q) : *reinterpret_cast<const f32x4*>(xr + 4 * q);
+        if (yr) {
+            const f32x4 z = load_quad(yr + 4 * q), w = *reinterpret_cast<const f32x4*>(y_w + 4 * q);
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v[r] += z[r] * yi * w[r];
+        }
+        if (step) {
+            const f32x4 z = *reinterpret_cast<const f32x4*>(step + 4 * q);
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v[r] += z[r];
+        }
+        s += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+        if (er || yr || step) *reinterpret_cast<f32x4*>(xr + 4 * q) = v;
+    }
+    s = block_sum256(s, red);
+    const float inv = 1.0f / sqrtf(s / (float)width_real + eps);
+    for (int q = threadIdx.x; q < nq; q += 256) {             // (each thread re-reads what it wrote itself)
+        f32x4 v = *reinterpret_cast<const f32x4*>(xr + 4 * q);
+        const f32x4 w = *reinterpret_cast<const f32x4*>(norm_w + 4 * q);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) v[r] = v[r] * inv * w[r];
+        store_quad(h + (int64_t)row * width + 4 * q, v);
+    }
+}
+
+extern "C" int tfl_finish(const void* embed, const int64_t* ids, int vocab, const void* y, int y_f32, int64_t ld_y,
+                          const float* y_w, const float* step, const float* norm_w, float* x, void* h, int rows, int width,
+                          int width_real, float eps, int dtype, void* stream) {
+    if (!x || !h || !norm_w || rows < 1 || width < 4 || (width & 3) || width_real < 1 || width_real > width) return TF_EINVAL;
+    if (embed && (!ids || vocab < 1)) return TF_EINVAL;
+    if (y && (!y_w || ld_y < width || (ld_y & 3))) return TF_EINVAL;
+    hipStream_t st = (hipStream_t)stream;
+#define GO(T, Y) hipLaunchKernelGGL((finish_kernel<T, Y>), dim3(rows), dim3(256), 0, st, (const T*)embed, ids, vocab, (const Y*)y, \
+                                    ld_y, y_w, step, norm_w, x, (T*)h, width, width_real, eps)
+    if (dtype == 0) { if (y_f32) GO(bf16, float); else GO(bf16, bf16); }
+    else if (dtype == 1) GO(float, float);
+    else return TF_EINVAL;
+#undef GO
+    TFL_LAUNCH_CHECK();
+    return TF_OK;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void residual_kernel(const T* __restrict__ d, float* __restrict__ x, T* __restrict__ xt,
+                                                       int64_t nq) {
+    for (int64_t q = (int64_t)blockIdx.x * 256 + threadIdx.x; q < nq; q += (int64_t)gridDim.x * 256) {
+        f32x4 v = *reinterpret_cast<const f32x4*>(x + 4 * q);
+        const f32x4 z = load_quad(d + 4 * q);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) v[r] += z[r];
+        *reinterpret_cast<f32x4*>(x + 4 * q) = v;
+        if (xt) store_quad(xt + 4 * q, v);
+    }
+}
+
+extern "C" int tfl_residual(const void* d, float* x, void* xt, int64_t n, int dtype, void* stream) {
+    if (!d || !x || n < 4 || (n & 3)) return TF_EINVAL;
+    const int64_t nq = n / 4;
+    const unsigned gx = (unsigned)((nq + 255) / 256 < 4096 ? (nq + 255) / 256 : 4096);
+    hipStream_t st = (hipStream_t)stream;
+    if (dtype == 0) hipLaunchKernelGGL((residual_kernel<bf16>), dim3(gx), dim3(256), 0, st, (const bf16*)d, x, (bf16*)xt, nq);
+    else if (dtype == 1) hipLaunchKernelGGL((residual_kernel<float>), dim3(gx), dim3(256), 0, st, (const float*)d, x, (float*)xt, nq);
+    else return TF_EINVAL;
+    TFL_LAUNCH_CHECK();
+    return TF_OK;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void token_gate_kernel(const T* __restrict__ s, int64_t ld_s, const T* __restrict__ table,
+                                                         int64_t ld_tok, const int64_t* __restrict__ ids, int vocab,
+                                                         T* __restrict__ out, int n, int n_real) {
+    const int row = blockIdx.x;
+    int64_t id = ids[row];
+    id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+    for (int c = threadIdx.x; c < n; c += 256)
+        out[(int64_t)row * n + c] = c < n_real ? (T)(gelu_tanh((float)s[(int64_t)row * ld_s + c]) * (float)table[id * ld_tok + c]) : (T)0.f;
+}
+
+extern "C" int tfl_token_gate(const void* s, int64_t ld_s, const void* table, int64_t ld_tok, const int64_t* ids, int vocab,
+                              void* out, int rows, int n, int n_real, int dtype, void* stream) {
+    if (!s || !table || !ids || !out || rows < 1 || n < 1 || n_real < 1 || n_real > n || ld_s < n || ld_tok < n_real || vocab < 1)
+        return TF_EINVAL;
+    hipStream_t st = (hipStream_t)stream;
+#define GO(T) hipLaunchKernelGGL((token_gate_kernel<T>), dim3(rows), dim3(256), 0, st, (const T*)s, ld_s, (const T*)table, ld_tok, \
+                                 ids, vocab, (T*)out, n, n_real)
+    if (dtype == 0) GO(bf16);
+    else if (dtype == 1) GO(float);
+    else return TF_EINVAL;
+#undef GO
+    TFL_LAUNCH_CHECK();
+    return TF_OK;
+}
+
+// One workgroup per new token.
+template <typename T>
+__global__ __launch_bounds__(256) void prepare_kernel(const T* __restrict__ y, int64_t ld_y, int q, int q_real, int C, int c_real,
+                                                      int R, int up_off, int n_up, const float* __restrict__ q_norm,
+                                                      const float* __restrict__ kv_norm, float eps, const float* __restrict__ cosb,
+                                                      const float* __restrict__ sinb, int half, int max_pos,
+                                                      const int32_t* __restrict__ pos, const int32_t* __restrict__ slot,
+                                                      T* __restrict__ cache, int cache_rows, T* __restrict__ cq, T* __restrict__ ck,
+                                                      T* __restrict__ act, int64_t ld_act) {
+    __shared__ float red[4];
+    const int row = blockIdx.x;
+    const T* yr = y + (int64_t)row * ld_y;
+    float s = 0.f;
+    for (int c = threadIdx.x; c < q / 4; c += 256) {
+        const f32x4 v = load_quad(yr + 4 * c);
+        s += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+    }
+    s = block_sum256(s, red);
+    const float inv = 1.0f / sqrtf(s / (float)q_real + eps);
+    for (int c = threadIdx.x; c < q / 4; c += 256) {
+        f32x4 v = load_quad(yr + 4 * c);
+        const f32x4 w = *reinterpret_cast<const f32x4*>(q_norm + 4 * c);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) v[r] = v[r] * inv * w[r];
+        store_quad(cq + (int64_t)row * q + 4 * c, v);
+    }
+    int p = pos[row];
+    p = p < 0 ? 0 : (p >= max_pos ? max_pos - 1 : p);
+    const int sl = slot[row], W = C + R;
+    const T* kv = yr + q;
+    cache_row_256<T>([kv](int c) { return (float)kv[c]; }, C, c_real, R, kv_norm, eps, cosb + (int64_t)p * half,
+                     sinb + (int64_t)p * half, half, sl >= 0 && sl < cache_rows ? cache + (int64_t)sl * W : (T*)nullptr,
+                     ck ? ck + (int64_t)row * W : (T*)nullptr, red);
+    for (int c = threadIdx.x; c < n_up / 4; c += 256) {
+        f32x4 v = load_quad(yr + up_off + 4 * c);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) v[r] = gelu_tanh(v[r]);
+        store_quad(act + (int64_t)row * ld_act + 4 * c, v);
+    }
+}
+
+extern "C" int tfl_prepare(const void* y, int64_t ld_y, int q, int q_real, int C, int c_real, int R, int up_off, int n_up,
+                           const float* q_norm, const float* kv_norm, float eps, const float* cosb, const float* sinb, int half,
+                           int max_pos, const int32_t* pos, const int32_t* slot, void* cache, int cache_rows, void* cq, void* ck,
+                           void* act, int64_t ld_act, int rows, int dtype, void* stream) {
+    if (!y || !q_norm || !kv_norm || !pos || !slot || !cache || !cq || rows < 1 || cache_rows < 1) return TF_EINVAL;
+    if (q < 4 || (q & 3) || q_real < 1 || q_real > q || C < 4 || (C & 3) || c_real < 1 || c_real > C || R < 0 || (R & 3)) return TF_EINVAL;
+    if (ld_y < q + C + R || (ld_y & 3) || half < 0 || 2 * half > R || max_pos < 1 || (half && (!cosb || !sinb))) return TF_EINVAL;
+    if (n_up < 0 || (n_up & 3) || (n_up && (!act || (ld_act & 3) || ld_act < n_up || (up_off & 3) || up_off < q + C + R || ld_y < up_off + n_up)))
+        return TF_EINVAL;
+    hipStream_t st = (hipStream_t)stream;
+#define GO(T) hipLaunchKernelGGL((prepare_kernel<T>), dim3(rows), dim3(256), 0, st, (const T*)y, ld_y, q, q_real, C, c_real, R, up_off, \
+                                 n_up, q_norm, kv_norm, eps, cosb, sinb, half, max_pos, pos, slot, (T*)cache, cache_rows, (T*)cq, \
+                                 (T*)ck, (T*)act, ld_act)
+    if (dtype == 0) GO(bf16);
+    else if (dtype == 1) GO(float);
+    else return TF_EINVAL;
+#undef GO
+    TFL_LAUNCH_CHECK();
+    return TF_OK;
+}
+
+// 16-byte pieces; a row is ppr of them.
+__global__ __launch_bounds__(256) void gather_rows_kernel(const uint4* __restrict__ cache, int cache_rows,
+                                                          const int32_t* __restrict__ src, uint4* __restrict__ dst, int rows, int ppr) {
+    const int64_t total = (int64_t)rows * ppr;
+    for (int64_t p = (int64_t)blockIdx.x * 256 + threadIdx.x; p < total; p += (int64_t)gridDim.x * 256) {
+        const int64_t r = p / ppr;
+        int s = src[r];
+        s = s < 0 ? 0 : (s >= cache_rows ? cache_rows - 1 : s);
+        dst[p] = cache[(int64_t)s * ppr + (p - r * ppr)];
+    }
+}
+
+extern "C" int tfl_gather_rows(const void* cache, int cache_rows, const int32_t* src, void* dst, int rows, int W, int dtype, void* stream) {
+    if (!cache || !src || !dst || rows < 1 || cache_rows < 1 || W < 8 || (W & 7) || (dtype != 0 && dtype != 1)) return TF_EINVAL;
+    const int ppr = W * (dtype ? 4 : 2) / 16;
+    const int64_t total = (int64_t)rows * ppr;
+    const unsigned gx = (unsigned)((total + 255) / 256 < 8192 ? (total + 255) / 256 : 8192);
+    hipLaunchKernelGGL(gather_rows_kernel, dim3(gx), dim3(256), 0, (hipStream_t)stream, (const uint4*)cache, cache_rows, src,
+                       (uint4*)dst, rows, ppr);
+    TFL_LAUNCH_CHECK();
+    return TF_OK;
+}
+
+__global__ void decode_prep_kernel(int32_t* __restrict__ len, const int32_t* __restrict__ table, int table_ld, int table_cols,
+                                   int32_t* __restrict__ pos, int32_t* __restrict__ slot, int32_t* __restrict__ klen, int rows) {
+    const int m = blockIdx.x * blockDim.x + threadIdx.x;
+    if (m >= rows) return;
+    const int l = len[m];
+    const bool live = l >= 0 && l / TFL_PAGE < table_cols;
+    pos[m] = live ? l : 0;
+    slot[m] = live ? table[(int64_t)m * table_ld + l / TFL_PAGE] * TFL_PAGE + l % TFL_PAGE : -1;
+    klen[m] = live ? l + 1 : 0;
+    if (live) len[m] = l + 1;
+}
+
+extern "C" int tfl_decode_prep(int32_t* len, const int32_t* table, int table_ld, int table_cols, int32_t* pos, int32_t* slot,
+                               int32_t* klen, int rows, void* stream) {
+    if (!len || !table || !pos || !slot || !klen || rows < 1 || table_cols < 1 || table_ld < table_cols) return TF_EINVAL;
+    hipLaunchKernelGGL(decode_prep_kernel, dim3((rows + 63) / 64), dim3(64), 0, (hipStream_t)stream, len, table, table_ld, table_cols,
+                       pos, slot, klen, rows);
+    TFL_LAUNCH_CHECK();
+    return TF_OK;
+}

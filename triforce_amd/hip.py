@@ -1,4 +1,5 @@
-"""ctypes binding of libtriforce_hip.so (C ABI in include/triforce_hip.h).
+"""ctypes binding of libtriforce_hip.so (C ABI in include/triforce_hip.h) and of libtriforce_latent.so
+(include/triforce_latent.h, ``latent_lib``).
 
 There is deliberately NO fallback: if the shared library is missing or a symbol is absent the
 import of any op raises.  Build it with ``python -m triforce_amd.build`` (hipcc, gfx950).
@@ -6,7 +7,7 @@ import of any op raises.  Build it with ``python -m triforce_amd.build`` (hipcc,
 import ctypes
 import os
 
-from .build import LIB_PATH
+from .build import LATENT_LIB_PATH, LIB_PATH
 
 _c = ctypes
 _vp, _i32, _i64, _f32 = _c.c_void_p, _c.c_int, _c.c_int64, _c.c_float
@@ -139,6 +140,41 @@ SIGNATURES["tf_draft_persist_reset"] = (_i32, [_vp, _vp, _i32])
 ABI_VERSION = 1
 _lib = None
 
+# ---- libtriforce_latent.so (include/triforce_latent.h) ------------------------------------------------------------------
+TFL_PAGE = 64
+TFL_EPI = {n: i for i, n in enumerate(("f32", "in", "query", "latent", "gated", "residual", "token"))}
+TFL_X = {"t": 0, "f32": 1, "f32_norm": 2}
+
+
+class TflGemm(_c.Structure):
+    """include/triforce_latent.h: TflGemm."""
+    _fields_ = ([(n, _vp) for n in ("wp", "x", "norm_w", "ss_in", "out_t", "out_t2", "out_f", "ss_out", "gate", "tok_table", "ids",
+                                    "pos", "cos", "sin", "kv_raw", "kv_norm_w", "cache", "slot")]
+                + [(n, _i64) for n in ("ld_x", "x_group", "ld_t", "ld_f", "ld_gate", "ld_tok", "ld_kv")]
+                + [(n, _i32) for n in ("rows", "n", "k", "groups", "n_real", "k_real", "n_raw", "ss_n", "ss_ld", "H", "N", "R", "C",
+                                       "half", "c_real", "max_pos", "cache_rows", "vocab")]
+                + [("eps", _f32)])
+
+
+LATENT_SIGNATURES = {
+    "tfl_abi_version": (_i32, []),
+    "tfl_gemm": (_i32, [_c.POINTER(TflGemm), _i32, _i32, _i32, _vp]),
+    "tfl_finish": (_i32, [_vp, _vp, _i32, _vp, _i32, _i64, _vp, _vp, _vp, _vp, _vp, _i32, _i32, _i32, _f32, _i32, _vp]),
+    "tfl_residual": (_i32, [_vp, _vp, _vp, _i64, _i32, _vp]),
+    "tfl_token_gate": (_i32, [_vp, _i64, _vp, _i64, _vp, _i32, _vp, _i32, _i32, _i32, _i32, _vp]),
+    "tfl_prepare": (_i32, [_vp, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _vp, _vp, _f32, _vp, _vp, _i32, _i32, _vp, _vp,
+                           _vp, _i32, _vp, _vp, _vp, _i64, _i32, _i32, _vp]),
+    "tfl_gather_rows": (_i32, [_vp, _i32, _vp, _vp, _i32, _i32, _i32, _vp]),
+    "tfl_attn_prefill": (_i32, [_vp, _vp, _vp, _vp, _i32, _i32, _vp, _vp, _vp, _i32, _i32, _vp, _i64, _vp, _i64, _i32, _i32, _i32,
+                                _i32, _i32, _i32, _i32, _f32, _i32, _vp]),
+    "tfl_attn_decode_ws_floats": (_i64, [_i32, _i32, _i32, _i32]),
+    "tfl_attn_decode_pick_nsplit": (_i32, [_i32, _i32, _i32]),
+    "tfl_attn_decode": (_i32, [_vp, _vp, _i32, _vp, _i32, _vp, _vp, _vp, _i64, _i32, _i32, _i32, _i32, _f32, _i32, _i32, _vp]),
+    "tfl_decode_prep": (_i32, [_vp, _vp, _i32, _i32, _vp, _vp, _vp, _i32, _vp]),
+}
+LATENT_ABI_VERSION = 1
+_latent = None
+
 
 class TriforceHipError(RuntimeError):
     pass
@@ -155,27 +191,40 @@ def _preload_torch_hip_runtime():
         ctypes.CDLL(cand, mode=ctypes.RTLD_GLOBAL)
 
 
+def _load(path, signatures, version_fn, version):
+    """Open a library and bind its entry points; raises (never falls back) when anything is missing."""
+    _preload_torch_hip_runtime()
+    if not os.path.exists(path):
+        raise TriforceHipError(
+            f"{path} not found: the HIP extension is required (python -m triforce_amd.build); "
+            "there is no CPU fallback")
+    L = ctypes.CDLL(path)
+    for name, (res, args) in signatures.items():
+        try:
+            fn = getattr(L, name)
+        except AttributeError as e:
+            raise TriforceHipError(f"{path} does not export {name}") from e
+        fn.restype, fn.argtypes = res, args
+    have = getattr(L, version_fn)()
+    if have != version:
+        raise TriforceHipError(f"ABI mismatch: library {have} != binding {version}")
+    return L
+
+
 def lib():
-    """The loaded library; raises (never falls back) when it cannot be loaded."""
+    """The core library."""
     global _lib
-    if _lib is None:
-        _preload_torch_hip_runtime()
-        path = os.environ.get("TRIFORCE_HIP_LIB", LIB_PATH)        # tuning builds (triforce_amd.build.build_variant)
-        if not os.path.exists(path):
-            raise TriforceHipError(
-                f"{path} not found: the HIP extension is required (python -m triforce_amd.build); "
-                "there is no CPU fallback")
-        L = ctypes.CDLL(path)
-        for name, (res, args) in SIGNATURES.items():
-            try:
-                fn = getattr(L, name)
-            except AttributeError as e:
-                raise TriforceHipError(f"{path} does not export {name}") from e
-            fn.restype, fn.argtypes = res, args
-        if L.tf_abi_version() != ABI_VERSION:
-            raise TriforceHipError(f"ABI mismatch: library {L.tf_abi_version()} != binding {ABI_VERSION}")
-        _lib = L
+    if _lib is None:                                               # TRIFORCE_HIP_LIB: tuning builds (triforce_amd.build.build_variant)
+        _lib = _load(os.environ.get("TRIFORCE_HIP_LIB", LIB_PATH), SIGNATURES, "tf_abi_version", ABI_VERSION)
     return _lib
+
+
+def latent_lib():
+    """The latent-attention library."""
+    global _latent
+    if _latent is None:
+        _latent = _load(LATENT_LIB_PATH, LATENT_SIGNATURES, "tfl_abi_version", LATENT_ABI_VERSION)
+    return _latent
 
 
 def check(rc, what):

@@ -15,7 +15,7 @@ from typing import Tuple
 
 import torch
 
-from .. import ops
+from .. import hip, ops
 
 
 class Cache:
@@ -561,3 +561,129 @@ class DistributedRetrievalCache_Seqouia(DistributedRetrievalCache):
         self.k[layer_idx].index_copy_(1, ids, k.permute(1, 0, 2).contiguous())
         self.v[layer_idx].index_copy_(1, ids, v.permute(1, 0, 2).contiguous())
         return self.key_cache[layer_idx], self.value_cache[layer_idx]
+
+
+# =============================================================================================
+# Latent cache (models/modeling_befidra.py): batches of sequences, pages of 64 rows
+# =============================================================================================
+class LatentBatch:
+    """What one forward over several sequences needs besides the token ids; device tensors unless said otherwise.
+
+    decode (one token per sequence): pos / slot / klen int32 [B], table int32 [B, columns], max_len (host int).
+    prefill: pos / slot int32 [tokens]; seq int32 [sequences, 4] = first new token, new tokens, first key, keys; max_new;
+    key_rows int32 [keys] = cache rows of every visible key, or None when no sequence has a past.
+    want: rows whose logits are asked for (int64), None = all."""
+
+    def __init__(self, decode, pos, slot, want=None, table=None, klen=None, max_len=0, seq=None, max_new=0, key_rows=None):
+        self.decode, self.pos, self.slot, self.want = decode, pos, slot, want
+        self.table, self.klen, self.max_len = table, klen, max_len
+        self.seq, self.max_new, self.key_rows = seq, max_new, key_rows
+
+
+class LatentCache(Cache):
+    """Latent + rotated-key rows of a batch of sequences.  Each layer run has one [pages * 64, row] block; a sequence owns whole
+    pages and gives them back in ``release``.  ``max_budget`` counts tokens of all live sequences together; every sequence may
+    leave its last page part-filled, so there is one spare page per sequence beyond that."""
+
+    DEFAULT = "sequence"                            # the sequence of the single-sequence entry points
+
+    def __init__(self, model, max_budget=1024, max_batch=64) -> None:
+        self.page = hip.TFL_PAGE
+        self.max_budget, self.max_batch = int(max_budget), int(max_batch)
+        if self.max_budget < 1 or self.max_batch < 1:
+            raise ValueError("max_budget and max_batch must be positive")
+        self.device = model.device
+        self.n_pages = -(-self.max_budget // self.page) + self.max_batch - 1
+        self.columns = -(-self.max_budget // self.page)              # a single sequence may hold the whole budget
+        self.rows = [torch.zeros(self.n_pages * self.page, w, dtype=model.dtype, device=self.device) for w in model.cache_widths()]
+        model.prepare_positions(self.max_budget)
+        self.generation = 0                         # bumped when a page is handed out or taken back (device tables go stale)
+        self.free, self.pages, self.length = [], {}, {}
+        self.reset()
+
+    # -- sequences -----------------------------------------------------------------------------
+    def reset(self):
+        self.free = list(range(self.n_pages - 1, -1, -1))
+        self.pages, self.length = {}, {}
+        self.generation += 1
+
+    @property
+    def seq_len(self):
+        return self.length.get(self.DEFAULT, 0)
+
+    @property
+    def tokens(self):
+        return sum(self.length.values())
+
+    def print_status(self):
+        print("[Latent Cache] Cached:", self.tokens, "| Budget:", self.max_budget, "| Sequences:", len(self.length), "| Free pages:",
+              len(self.free), "of", self.n_pages)
+
+    def release(self, seq):
+        """The sequence is finished: its pages are free for others."""
+        self.free.extend(reversed(self.pages.pop(seq)))
+        del self.length[seq]
+        self.generation += 1
+
+    def extend(self, wants):
+        """Room for the new tokens of a step ([(sequence, n)]), all of it or none: raises IndexError when the budget, the batch
+        limit or the pages do not allow it.  Lengths advance."""
+        fresh = [s for s, _ in wants if s not in self.length]
+        if self.tokens + sum(n for _, n in wants) > self.max_budget:
+            raise IndexError(f"LatentCache overflow: {self.tokens} + {sum(n for _, n in wants)} > {self.max_budget} tokens")
+        if len(self.length) + len(fresh) > self.max_batch:
+            raise IndexError(f"LatentCache: {len(self.length) + len(fresh)} sequences > {self.max_batch}")
+        for s, n in wants:
+            if s not in self.length:
+                self.length[s], self.pages[s] = 0, []
+            self.length[s] += n
+            need = -(-self.length[s] // self.page) - len(self.pages[s])
+            for _ in range(need):
+                self.pages[s].append(self.free.pop())
+            if need:
+                self.generation += 1
+
+    def cache_rows(self, seq, first, n):
+        """Cache row of tokens first .. first + n - 1 of a sequence (int32 CPU tensor)."""
+        pages = torch.tensor(self.pages[seq], dtype=torch.int32)
+        t = torch.arange(first, first + n)
+        return pages[t // self.page] * self.page + (t % self.page).to(torch.int32)
+
+    # -- batch descriptions --------------------------------------------------------------------
+    def _send(self, parts):
+        """CPU int32 tensors -> device views of one transfer."""
+        flat = torch.cat([p.reshape(-1) for p in parts]).to(self.device)
+        out, at = [], 0
+        for p in parts:
+            out.append(flat[at:at + p.numel()].view(p.shape))
+            at += p.numel()
+        return out
+
+    def plan_prefill(self, entries):
+        """entries: [(sequence, new tokens, wanted places among them)] -> LatentBatch; the sequences grow by the new tokens."""
+        past = {s: self.length.get(s, 0) for s, _, _ in entries}
+        self.extend([(s, n) for s, n, _ in entries])
+        pos, slot, seq, key_rows, want = [], [], [], [], []
+        q_at = k_at = 0
+        for s, n, w in entries:
+            p = past[s]
+            pos.append(torch.arange(p, p + n, dtype=torch.int32))
+            rows = self.cache_rows(s, 0, p + n)
+            slot.append(rows[p:])
+            key_rows.append(rows)
+            seq.append((q_at, n, k_at, p + n))
+            want += [q_at + j for j in w]
+            q_at, k_at = q_at + n, k_at + p + n
+        any_past = any(past.values())
+        parts = [torch.cat(pos), torch.cat(slot), torch.tensor(seq, dtype=torch.int32)] + ([torch.cat(key_rows)] if any_past else [])
+        dev = self._send(parts)
+        w = None if len(want) == q_at else torch.tensor(want, dtype=torch.int64).to(self.device)
+        return LatentBatch(False, dev[0], dev[1], want=w, seq=dev[2], max_new=max(n for _, n, _ in entries),
+                           key_rows=dev[3] if any_past else None)
+
+    def tables(self, seqs):
+        """(lengths int32 [B], page tables int32 [B, columns]) of some sequences, on the CPU; unused columns are 0."""
+        table = torch.zeros(len(seqs), self.columns, dtype=torch.int32)
+        for b, s in enumerate(seqs):
+            table[b, :len(self.pages[s])] = torch.tensor(self.pages[s], dtype=torch.int32)
+        return torch.tensor([self.length[s] for s in seqs], dtype=torch.int32), table

@@ -1,0 +1,122 @@
+"""Configuration of the Befidra design: parallel layers (one norm, mixer and feed-forward both read it) with latent attention,
+a range of layers that is run several times, and a per-layer input from a second embedding table.
+
+``config.json`` keys: vocab, width, norm.eps, layers[] (type, mixer, mlp | null), loop (start, stop, times; optional),
+token_side.dim (optional).  Every size and constant is per model, most of them per layer.
+"""
+import json
+import os
+
+ARCHITECTURE = "Befidra"
+
+
+class RotarySpec:
+    """Interleaved rotary positions: dims, base and optional YaRN scaling (factor, original, fast, slow)."""
+
+    def __init__(self, dims, base, scaling=None):
+        self.dims, self.base = int(dims), float(base)
+        if self.dims < 0 or self.dims % 2:
+            raise ValueError(f"rot.dims must be even, got {dims}")
+        self.scaling = None
+        if scaling is not None:
+            missing = [k for k in ("factor", "original", "fast", "slow") if k not in scaling]
+            if missing:
+                raise ValueError(f"rot.scaling lacks {missing}")
+            self.scaling = {k: float(scaling[k]) for k in ("factor", "original", "fast", "slow")}
+
+    def key(self):
+        s = self.scaling
+        return (self.dims, self.base) + (() if s is None else (s["factor"], s["original"], s["fast"], s["slow"]))
+
+    def to_dict(self):
+        d = {"dims": self.dims, "base": self.base}
+        if self.scaling is not None:
+            d["scaling"] = dict(self.scaling)
+        return d
+
+
+class LatentMixerSpec:
+    """Sizes of one latent-attention mixer."""
+    FIELDS = ("heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank")
+
+    def __init__(self, d):
+        for k in self.FIELDS:
+            v = int(d[k])
+            if v < 1:
+                raise ValueError(f"mixer.{k} must be positive, got {v}")
+            setattr(self, k, v)
+        self.scale = float(d["scale"])
+        self.rot = RotarySpec(**d["rot"])
+        if self.rot.dims > self.rot_dim:
+            raise ValueError("rot.dims exceeds rot_dim")
+
+    def to_dict(self):
+        return dict({k: getattr(self, k) for k in self.FIELDS}, scale=self.scale, rot=self.rot.to_dict())
+
+
+class LayerSpec:
+    def __init__(self, d):
+        if d["type"] != "latent_attention":
+            raise ValueError(f"unknown mixer type {d['type']!r}")
+        self.type = d["type"]
+        self.mixer = LatentMixerSpec(d["mixer"])
+        mlp = d.get("mlp")
+        if mlp is not None and mlp.get("kind") != "dense":
+            raise ValueError(f"unknown feed-forward kind {mlp.get('kind')!r}")
+        self.ff = 0 if mlp is None else int(mlp["ff"])
+
+    def to_dict(self):
+        return {"type": self.type, "mixer": self.mixer.to_dict(), "mlp": {"kind": "dense", "ff": self.ff} if self.ff else None}
+
+
+class BefidraConfig:
+    def __init__(self, vocab, width, layers, norm, loop=None, token_side=None, _name_or_path="", eos_token_id=None, **_):
+        self.vocab_size, self.hidden_size = int(vocab), int(width)
+        self.layers = [LayerSpec(d) for d in layers]
+        self.eps = float(norm["eps"])
+        self.loop = None if loop is None else (int(loop["start"]), int(loop["stop"]), int(loop["times"]))
+        if self.loop is not None:
+            a, b, n = self.loop
+            if not (0 <= a < b <= len(self.layers) and n >= 1):
+                raise ValueError(f"loop {self.loop} does not fit {len(self.layers)} layers")
+        self.side_dim = 0 if token_side is None else int(token_side["dim"])
+        self._name_or_path, self.eos_token_id = _name_or_path, eos_token_id
+        if not self.layers:
+            raise ValueError("no layers")
+
+    @property
+    def num_hidden_layers(self):
+        return len(self.layers)
+
+    def layer_runs(self):
+        """(layer, pass of the loop or None, does a pass start here) in execution order; each entry has a cache of its own."""
+        n = len(self.layers)
+        if self.loop is None:
+            return [(i, None, False) for i in range(n)]
+        a, b, times = self.loop
+        runs = [(i, None, False) for i in range(a)]
+        for t in range(times):
+            runs += [(i, t, i == a) for i in range(a, b)]
+        return runs + [(i, None, False) for i in range(b, n)]
+
+    @classmethod
+    def from_dict(cls, d):
+        d = dict(d)
+        d.pop("architecture", None)
+        return cls(**d)
+
+    @classmethod
+    def from_pretrained(cls, path):
+        with open(os.path.join(path, "config.json")) as f:
+            d = json.load(f)
+        d["_name_or_path"] = path
+        return cls.from_dict(d)
+
+    def to_dict(self):
+        d = {"architecture": ARCHITECTURE, "vocab": self.vocab_size, "width": self.hidden_size, "norm": {"eps": self.eps},
+             "layers": [s.to_dict() for s in self.layers]}
+        if self.loop is not None:
+            d["loop"] = dict(zip(("start", "stop", "times"), self.loop))
+        if self.side_dim:
+            d["token_side"] = {"dim": self.side_dim}
+        return d

@@ -1,0 +1,215 @@
+"""Weights, rotary tables and the per-layer compute of a latent-attention decoder on the HIP ops (ops_latent).
+
+Decode form of a layer (one token per sequence, any number of sequences): ten launches - [norm] [input projections, gelu]
+[query up-projection + cache append] [query to latent] [attention, merge] [latent to value, gate] [output + feed-forward down,
+residual] [token gate] [token projection].  Prefill form: library GEMMs between the row kernels and the up-projected attention.
+"""
+import math
+import zlib
+
+import torch
+
+from .. import ops_latent as ol
+
+
+def rotary_frequencies(spec):
+    """fp64 frequencies of the rotation pairs and the factor on cos / sin (YaRN: interpolated below a ramp, stretched above)."""
+    n = spec.dims
+    f = [spec.base ** (-2.0 * i / n) for i in range(n // 2)]
+    s = spec.scaling
+    if s is None:
+        return f, 1.0
+
+    def dim_of(turns):                                # the dimension that makes ``turns`` turns over the original context
+        return n * math.log(s["original"] / (2.0 * math.pi * turns)) / (2.0 * math.log(spec.base))
+    lo, hi = max(math.floor(dim_of(s["fast"])), 0), min(math.ceil(dim_of(s["slow"])), n - 1)
+    out = []
+    for i, x in enumerate(f):
+        ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+        out.append(x / s["factor"] * ramp + x * (1.0 - ramp))
+    return out, 0.1 * math.log(s["factor"]) + 1.0
+
+
+class RotaryTable:
+    """cos / sin of every position, fp32 [max_pos, pairs] (angles and functions in fp64 before the one rounding)."""
+
+    def __init__(self, spec, max_pos, device):
+        f, m = rotary_frequencies(spec)
+        self.half, self.max_pos = len(f), int(max_pos)
+        a = torch.arange(self.max_pos, dtype=torch.float64)[:, None] * torch.tensor(f, dtype=torch.float64)[None, :]
+        self.cos = (a.cos() * m).to(torch.float32).contiguous().to(device)
+        self.sin = (a.sin() * m).to(torch.float32).contiguous().to(device)
+
+
+class LatentGeom:
+    """Sizes of one latent mixer padded to multiples of 32 (H heads, N / R unrotated / rotated query-key size, V value size,
+    C latent, Q query latent) next to the real ones the norms divide by."""
+
+    def __init__(self, m):
+        p = ol.pad32
+        self.H, self.N, self.R, self.V, self.C, self.Q = m.heads, p(m.dim), p(m.rot_dim), p(m.vdim), p(m.kv_rank), p(m.q_rank)
+        self.c_real, self.q_real = m.kv_rank, m.q_rank
+
+    n_raw = property(lambda s: s.Q + s.C + s.R + s.H * s.V)       # fp32 part of the input projection
+    gate_off = property(lambda s: s.Q + s.C + s.R)
+    row = property(lambda s: s.C + s.R)                           # one cached row
+
+
+def _grow(t, *shape):
+    """Zero-pad the trailing edge of every dimension to ``shape``."""
+    if tuple(t.shape) == tuple(shape):
+        return t
+    out = torch.zeros(*shape, dtype=t.dtype, device=t.device)
+    out[tuple(slice(0, n) for n in t.shape)] = t
+    return out
+
+
+class LatentLayer:
+    """One layer's weights in the forms the kernels take."""
+
+    def __init__(self, spec, width, side_dim, get, dtype):
+        m, g, p = spec.mixer, LatentGeom(spec.mixer), ol.pad32
+        self.spec, self.geom, self.scale = spec, g, m.scale
+        W, F, D = p(width), p(spec.ff) if spec.ff else 0, p(side_dim) if side_dim else 0
+        self.width, self.ff, self.side_dim = W, F, side_dim
+
+        def vec(name, n):
+            return _grow(get(name).float(), n)
+
+        def mat(name):
+            return get(name).to(dtype)
+        dkv = mat("mix.dkv")
+        parts = [_grow(mat("mix.dq"), g.Q, W), _grow(dkv[:m.kv_rank], g.C, W), _grow(dkv[m.kv_rank:], g.R, W),
+                 _grow(mat("mix.g").view(g.H, m.vdim, width), g.H, g.V, W).reshape(g.H * g.V, W)]
+        if F:
+            parts.append(_grow(mat("mlp.up"), F, W))
+        self.w_in = ol.TileWeight(torch.cat(parts))
+        uq = mat("mix.uq").view(g.H, m.dim + m.rot_dim, m.q_rank)
+        self.w_uq = ol.TileWeight(torch.cat([_grow(uq[:, :m.dim], g.H, g.N, g.Q), _grow(uq[:, m.dim:], g.H, g.R, g.Q)], 1)
+                                  .reshape(g.H * (g.N + g.R), g.Q))
+        uk = _grow(mat("mix.uk").view(g.H, m.dim, m.kv_rank), g.H, g.N, g.C)
+        uv = _grow(mat("mix.uv").view(g.H, m.vdim, m.kv_rank), g.H, g.V, g.C)
+        self.w_uk_t = ol.TileWeight(uk.transpose(1, 2).contiguous(), packed_only=True)          # decode: query -> latent
+        self.w_uv = ol.TileWeight(uv, packed_only=True)                                         # decode: latent -> value
+        self.w_ukv = torch.cat([uk.reshape(g.H * g.N, g.C), uv.reshape(g.H * g.V, g.C)])        # prefill: keys | values
+        out = [_grow(mat("mix.o").view(width, g.H, m.vdim), W, g.H, g.V).reshape(W, g.H * g.V)]
+        if F:
+            out.append(_grow(mat("mlp.down"), W, F))
+        self.w_out = ol.TileWeight(torch.cat(out, 1))
+        self.norm1, self.q_norm, self.kv_norm = vec("norm1", W), vec("mix.dq.norm", g.Q), vec("mix.dkv.norm", g.C)
+        if D:
+            self.side_gate = ol.TileWeight(_grow(mat("side.gate"), D, W))
+            self.side_proj = ol.TileWeight(_grow(mat("side.proj"), W, D))
+            self.side_norm = vec("side.norm", W)
+
+    def weights(self):
+        return [self.w_in, self.w_uq, self.w_uk_t, self.w_uv, self.w_out] + ([self.side_gate, self.side_proj] if self.side_dim else [])
+
+    # -- the two forms of a layer: h (normed input), x (fp32 residual, updated) -> y (token-side output, added by the next norm) ----
+    def decode(self, h, x, ids, side_table, batch, rope, cache_rows, eps):
+        g = self.geom
+        act = torch.empty(h.shape[0], self.w_out.k, dtype=h.dtype, device=h.device)
+        raw, ss = ol.input_projection(h, self.w_in, g.n_raw, act, g.H * g.V)
+        qn, q = ol.query_and_append(raw, ss, self.w_uq, g, self.q_norm, self.kv_norm, eps, rope, batch.pos, batch.slot, cache_rows)
+        ol.query_to_latent(qn, self.w_uk_t, q, g)
+        o = ol.attn_decode(q, cache_rows, batch.table, batch.klen, g, self.scale, batch.max_len)
+        ol.latent_to_value(o, self.w_uv, raw, g.gate_off, act, g)
+        ol.add_linear(act, self.w_out, x)
+        if not self.side_dim:
+            return None
+        return ol.linear_f32(ol.token_gate_linear(x, self.side_gate, side_table, ids, self.side_dim), self.side_proj, self.width)
+
+    def prefill(self, h, x, ids, side_table, batch, rope, cache_rows, eps):
+        g = self.geom
+        act = torch.empty(h.shape[0], self.w_out.k, dtype=h.dtype, device=h.device)
+        y = self.w_in.matmul(h)
+        cq, ck = ol.prepare(y, g, g.n_raw, self.ff, self.q_norm, self.kv_norm, eps, rope, batch.pos, batch.slot, cache_rows, act,
+                            g.H * g.V, want_rows=batch.key_rows is None)
+        if ck is None:
+            ck = ol.gather_rows(cache_rows, batch.key_rows)              # earlier portions' rows and the ones just stored
+        q = self.w_uq.matmul(cq)
+        kv = torch.nn.functional.linear(ck[:, :g.C], self.w_ukv)
+        ol.attn_prefill(q, kv, ck, batch.seq, batch.max_new, batch.pos, rope, y[:, g.gate_off:], act, g, self.scale)
+        d = self.w_out.matmul(act)
+        xt = ol.residual(d, x, want_copy=bool(self.side_dim))
+        if not self.side_dim:
+            return None
+        return self.side_proj.matmul(ol.token_gate(self.side_gate.matmul(xt), side_table, ids, self.side_dim))
+
+
+class LatentWeights:
+    """Device-resident weights of the whole model in ``dtype`` (norm weights and loop steps fp32)."""
+
+    def __init__(self, cfg, device, dtype):
+        self.cfg, self.device, self.dtype = cfg, torch.device(device), dtype
+        self.layers = []
+        self.embed = self.logits = self.final_norm = self.side_embed = self.step = None
+        self.capture = None       # list -> the forward appends the residual stream after every layer run (comparisons)
+
+    def shapes(self):
+        """Tensor name -> shape of a checkpoint."""
+        c, d = self.cfg, self.cfg.hidden_size
+        out = {"embed": (c.vocab_size, d), "final.norm": (d,)}
+        if c.loop is not None:
+            out["loop.step"] = (c.loop[2], d)
+        if c.side_dim:
+            out["side.embed"] = (c.vocab_size, c.num_hidden_layers * c.side_dim)
+        for i, s in enumerate(c.layers):
+            m, p = s.mixer, f"l{i}."
+            out.update({p + "norm1": (d,), p + "mix.dq": (m.q_rank, d), p + "mix.dq.norm": (m.q_rank,),
+                        p + "mix.uq": (m.heads * (m.dim + m.rot_dim), m.q_rank), p + "mix.dkv": (m.kv_rank + m.rot_dim, d),
+                        p + "mix.dkv.norm": (m.kv_rank,), p + "mix.uk": (m.heads * m.dim, m.kv_rank),
+                        p + "mix.uv": (m.heads * m.vdim, m.kv_rank), p + "mix.g": (m.heads * m.vdim, d),
+                        p + "mix.o": (d, m.heads * m.vdim)})
+            if s.ff:
+                out.update({p + "mlp.up": (s.ff, d), p + "mlp.down": (d, s.ff)})
+            if c.side_dim:
+                out.update({p + "side.gate": (c.side_dim, d), p + "side.proj": (d, c.side_dim), p + "side.norm": (d,)})
+        return out
+
+    def _build(self, get):
+        c, d = self.cfg, ol.pad32(self.cfg.hidden_size)
+        embed = _grow(get("embed").to(self.dtype), c.vocab_size, d)
+        self.embed = embed.contiguous()
+        self.logits = ol.TileWeight(_grow(embed, ol.pad32(c.vocab_size), d), packed_only=True)
+        self.final_norm = _grow(get("final.norm").float(), d)
+        if c.loop is not None:
+            self.step = _grow(get("loop.step").float(), c.loop[2], d).contiguous()
+        if c.side_dim:
+            self.side_embed = get("side.embed").to(self.dtype).contiguous()
+        self.layers = [LatentLayer(s, c.hidden_size, c.side_dim, lambda n, i=i: get(f"l{i}." + n), self.dtype)
+                       for i, s in enumerate(c.layers)]
+        return self
+
+    def load_state_dict(self, sd):
+        want = self.shapes()
+        missing = [n for n in want if n not in sd]
+        if missing:
+            raise KeyError(f"checkpoint lacks {missing[:4]}{' ...' if len(missing) > 4 else ''}")
+        for n, s in want.items():
+            if tuple(sd[n].shape) != s:
+                raise ValueError(f"{n}: shape {tuple(sd[n].shape)}, the configuration says {s}")
+        return self._build(lambda n: sd[n].to(self.device))
+
+    def init_random(self, seed):
+        """Gaussian weights with 1 / sqrt(fan-in) scale, unit norms; one generator per tensor (order does not matter)."""
+        want = self.shapes()
+
+        def get(n):
+            s = want[n]
+            if n.endswith("norm") or n.endswith("norm1"):
+                return torch.ones(s, device=self.device)
+            g = torch.Generator(device=self.device)
+            g.manual_seed((seed * 1000003 + zlib.crc32(n.encode())) % (2 ** 31))
+            std = 1.0 if n == "side.embed" else (0.1 if n == "loop.step" else (0.02 if n == "embed" else s[1] ** -0.5))
+            return torch.randn(s, generator=g, device=self.device, dtype=torch.float32) * std
+        return self._build(get)
+
+    def side_table(self, i):
+        n = self.cfg.side_dim
+        return self.side_embed[:, i * n:(i + 1) * n] if n else None
+
+    def nbytes(self):
+        ts = [t for t in (self.embed, self.side_embed) if t is not None]
+        return sum(t.numel() * t.element_size() for t in ts) + sum(w.nbytes() for L in self.layers for w in L.weights()) \
+            + self.logits.nbytes()

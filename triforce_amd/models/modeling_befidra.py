@@ -1,0 +1,102 @@
+"""Befidra on the HIP ops: parallel layers over latent attention, a looped range of layers, per-layer token inputs.
+
+Same surface as the other target models (``from_pretrained`` / ``from_state_dict`` / ``init_random``, ``model(input_ids=,
+kv_cache=).logits`` for one sequence), plus ``forward_batch`` for a batch of sequences that is described by a
+``models.cache.LatentBatch``.  Residual stream, norms, rotation, softmax and gates are fp32; matrix products run in the model's
+dtype (bfloat16, or float32 throughout) with fp32 accumulation.
+"""
+import torch
+
+from .. import ops_latent as ol
+from .config_befidra import BefidraConfig
+from .latent_core import LatentWeights, RotaryTable
+from .llama_core import CausalLMOutput, load_checkpoint_state_dict, parse_random_spec
+
+
+class BefidraForCausalLM:
+    supports_speculation = False                   # no retrieval cache over latents: the engines serve it autoregressively
+
+    def __init__(self, config: BefidraConfig, device="cuda:0", dtype=torch.bfloat16):
+        if dtype not in (torch.bfloat16, torch.float32):
+            raise ValueError(f"dtype must be bfloat16 or float32, got {dtype}")
+        self.config, self.device, self.dtype = config, torch.device(device), dtype
+        self.vocab_size = config.vocab_size
+        self.weights = LatentWeights(config, self.device, dtype)
+        self.runs = config.layer_runs()
+        self._rope = {}
+        self.max_positions = 0
+
+    # -- construction ------------------------------------------------------------------------
+    @classmethod
+    def from_pretrained(cls, name_or_path, torch_dtype=torch.bfloat16, device_map="cuda:0", config=None, **_):
+        """Local checkpoint directory, or ``random:<seed>`` with an explicit ``config``."""
+        seed = parse_random_spec(name_or_path)
+        if seed is not None:
+            assert config is not None, "random:<seed> needs config="
+            return cls(config, device_map, torch_dtype).init_random(seed)
+        m = cls(config or BefidraConfig.from_pretrained(name_or_path), device_map, torch_dtype)
+        m.weights.load_state_dict(load_checkpoint_state_dict(name_or_path))
+        return m
+
+    @classmethod
+    def from_state_dict(cls, config, sd, device="cuda:0", dtype=torch.bfloat16):
+        m = cls(config, device, dtype)
+        m.weights.load_state_dict(sd)
+        return m
+
+    def init_random(self, seed):
+        self.weights.init_random(seed)
+        return self
+
+    def eval(self):
+        return self
+
+    # -- sizes the cache asks for ------------------------------------------------------------
+    def cache_widths(self):
+        """Elements of one cached row per layer run (every pass of a looped layer has a cache of its own)."""
+        from .latent_core import LatentGeom
+        return [LatentGeom(self.config.layers[i].mixer).row for i, _, _ in self.runs]
+
+    def prepare_positions(self, n):
+        """Rotary tables for positions 0 .. n-1 (called by the cache: captured graphs keep the tables' addresses)."""
+        if n > self.max_positions:
+            self.max_positions = n
+            specs = {s.mixer.rot.key(): s.mixer.rot for s in self.config.layers}
+            self._rope = {k: RotaryTable(s, n, self.device) for k, s in specs.items()}
+
+    # -- forward -----------------------------------------------------------------------------
+    @torch.inference_mode()
+    def __call__(self, input_ids, kv_cache=None, graph_cache=None, position_ids=None, **_):
+        return self.forward(input_ids, kv_cache)
+
+    def forward(self, input_ids, kv_cache, graph_cache=None, position_ids=None, last_rows=None):
+        """One sequence (the cache's default one), ``input_ids`` (1, n): appends n tokens, logits (1, rows, V) of the trailing
+        ``last_rows`` (default: all)."""
+        n = input_ids.shape[1]
+        want = range(n if last_rows is None else max(0, n - last_rows), n) if last_rows is not None else range(n)
+        batch = kv_cache.plan_prefill([(kv_cache.DEFAULT, n, want)])
+        return CausalLMOutput(self.forward_batch(input_ids.reshape(-1).to(self.device), batch, kv_cache).unsqueeze(0))
+
+    @torch.inference_mode()
+    def forward_batch(self, ids, batch, cache):
+        """ids int64 [tokens of the batch]; returns fp32 logits [wanted tokens, V] (None when nothing is wanted)."""
+        W, eps, width = self.weights, self.config.eps, self.config.hidden_size
+        x = torch.empty(ids.numel(), ol.pad32(width), dtype=torch.float32, device=self.device)
+        y = y_w = None
+        for r, (i, t, first) in enumerate(self.runs):
+            L = W.layers[i]
+            h = ol.finish(x, L.norm1, eps, width, self.dtype, embed=W.embed if r == 0 else None, ids=ids if r == 0 else None,
+                          y=y, y_w=y_w, step=W.step[t] if first else None)
+            if W.capture is not None and r > 0:
+                W.capture.append((x - W.step[t] if first else x.clone())[:, :width])
+            layer = L.decode if batch.decode else L.prefill
+            y = layer(h, x, ids, W.side_table(i), batch, self._rope[L.spec.mixer.rot.key()], cache.rows[r], eps)
+            y_w = L.side_norm if y is not None else None
+        if batch.want is not None and batch.want.numel() == 0:
+            return None
+        if batch.want is not None:
+            x, y = x[batch.want], None if y is None else y[batch.want]
+        h = ol.finish(x, W.final_norm, eps, width, self.dtype, y=y, y_w=y_w)
+        if W.capture is not None:
+            W.capture.append(x[:, :width].clone())
+        return ol.linear_f32(h, W.logits, self.vocab_size)

@@ -1,0 +1,43 @@
+"""Which configuration and model class serve a checkpoint: chosen by its config.json (``architecture``, or the first of
+``architectures``; a configuration that names none is a Llama, as the checkpoints of the speculative path are)."""
+import importlib
+import json
+import os
+
+# architecture -> (configuration module, class, model module, class)
+ARCHITECTURES = {
+    "LlamaForCausalLM": ("config_yarn", "LlamaConfig", "modeling_llama", "LlamaForCausalLM"),
+    "Befidra": ("config_befidra", "BefidraConfig", "modeling_befidra", "BefidraForCausalLM"),
+}
+
+
+def architecture_of(config):
+    """config: a dict, or a checkpoint directory."""
+    if not isinstance(config, dict):
+        with open(os.path.join(config, "config.json")) as f:
+            config = json.load(f)
+    name = config.get("architecture") or (config.get("architectures") or ["LlamaForCausalLM"])[0]
+    if name not in ARCHITECTURES:
+        raise NotImplementedError(f"unknown architecture {name!r}; known: {sorted(ARCHITECTURES)}")
+    return name
+
+
+def _load(module, name):
+    return getattr(importlib.import_module("." + module, __package__), name)
+
+
+def config_class(architecture):
+    return _load(*ARCHITECTURES[architecture][:2])
+
+
+def model_class(architecture):
+    return _load(*ARCHITECTURES[architecture][2:])
+
+
+def config_from_dict(d):
+    return config_class(architecture_of(d)).from_dict(d)
+
+
+def load_model(path, device, **kw):
+    """Checkpoint directory -> model on the device (``torch_dtype=`` where the architecture offers a choice)."""
+    return model_class(architecture_of(path)).from_pretrained(path, device_map=device, **kw)

@@ -1,9 +1,20 @@
 """Shapes of the models the TriForce entry points name (the reference hard-codes hub ids:
 test/on_chip.py:48-56, test/offloading_TP.py:56-67); offline they are built from these configs with
 random-init weights, or loaded from a local HF directory.  Values are the public model cards'."""
-from .config_yarn import LlamaConfig
+from . import registry
 
 _YARN_128K = dict(type="yarn", factor=32.0, original_max_position_embeddings=4096)
+
+
+
+def _befidra(name, width, ff, layers, loop, side, vocab, heads, dim, rot_dim, vdim, q_rank, kv_rank, base, scaling):
+    """A Befidra shape with equal layers (the configuration itself allows every layer its own sizes)."""
+    mixer = dict(heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim, q_rank=q_rank, kv_rank=kv_rank,
+                 scale=(dim + rot_dim) ** -0.5, rot=dict(dims=rot_dim, base=base, scaling=scaling))
+    return dict(architecture="Befidra", vocab=vocab, width=width, norm=dict(eps=1e-5), loop=loop, token_side=dict(dim=side),
+                layers=[dict(type="latent_attention", mixer=mixer, mlp=dict(kind="dense", ff=ff)) for _ in range(layers)],
+                _name_or_path=name)
+
 
 CONFIGS = {
     # NousResearch/Yarn-Llama-2-7b-128k
@@ -29,13 +40,20 @@ CONFIGS = {
                  max_position_embeddings=131072, rms_norm_eps=1e-6,
                  rope_scaling=dict(type="yarn", factor=16.0, original_max_position_embeddings=256),
                  _name_or_path="tiny-yarn-target"),
+    # Befidra: a 7B-like layer (32 heads over a 512 + 64 latent row), and a toy for smoke paths.  No public checkpoints.
+    "befidra-7B": _befidra("befidra-7b", width=4096, ff=11008, layers=32, loop=dict(start=8, stop=24, times=2), side=256, vocab=32000,
+                           heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512, base=10000.0,
+                           scaling=dict(factor=32.0, original=4096, fast=32.0, slow=1.0)),
+    "befidra-tiny": _befidra("befidra-tiny", width=192, ff=352, layers=3, loop=dict(start=1, stop=3, times=2), side=40, vocab=1000,
+                             heads=3, dim=48, rot_dim=24, vdim=40, q_rank=72, kv_rank=80, base=10000.0,
+                             scaling=dict(factor=8.0, original=256, fast=16.0, slow=2.0)),
 }
 
 
 def config(name):
     if name not in CONFIGS:
         raise NotImplementedError(f"unknown model {name!r}; known: {sorted(CONFIGS)}")
-    return LlamaConfig.from_dict(CONFIGS[name])
+    return registry.config_from_dict(CONFIGS[name])
 
 
 def find_checkpoint(name):

@@ -1,0 +1,270 @@
+"""Tensor-level wrappers over the latent-attention C ABI (include/triforce_latent.h).
+
+Same rules as ops.py: torch owns the memory and the stream, every function validates its tensors and enqueues hand-written
+gfx950 kernels on torch's current stream; no CPU path exists.  The element type is bfloat16 or float32 and follows the
+tensors.  Call these as ``ops_latent.<name>(...)``.
+"""
+import ctypes
+
+import torch
+import torch.nn.functional as F
+
+from . import hip
+
+PAGE = hip.TFL_PAGE
+_CODE = {torch.bfloat16: 0, torch.float32: 1}
+
+
+def pad32(n):
+    return (n + 31) // 32 * 32
+
+
+def _stream():
+    return ctypes.c_void_p(torch.cuda.current_stream().cuda_stream)
+
+
+def _p(t):
+    return None if t is None else ctypes.c_void_p(t.data_ptr())
+
+
+def _need(*ts):
+    for t in ts:
+        if t is not None:
+            if not t.is_cuda:
+                raise hip.TriforceHipError("triforce_amd ops need HIP device tensors (no CPU fallback)")
+            assert t.is_contiguous() or t.stride(-1) == 1
+
+
+def _f32(*ts):
+    assert all(t is None or t.dtype == torch.float32 for t in ts)
+
+
+def _i32(*ts):
+    assert all(t is None or t.dtype == torch.int32 for t in ts)
+
+
+def pack_tiles(w):
+    """[.., n, k] -> MFMA operand order [.., n/16, k/32, 4 (k octet), 16 (row), 8]: one 16x32 tile is one wavefront load."""
+    n, k = w.shape[-2:]
+    assert n % 16 == 0 and k % 32 == 0
+    lead = w.shape[:-2]
+    d = len(lead)
+    return w.reshape(*lead, n // 16, 16, k // 32, 4, 8).permute(*range(d), d, d + 2, d + 3, d + 1, d + 4).contiguous()
+
+
+class TileWeight:
+    """A (groups of) [n, k] weight(s): packed for the skinny kernel and, unless ``packed_only``, row-major for the library GEMM
+    of the prefill."""
+
+    def __init__(self, w, packed_only=False):
+        w3 = w if w.dim() == 3 else w.unsqueeze(0)
+        self.groups, self.n, self.k = w3.shape
+        self.packed = pack_tiles(w3)
+        self.w = None if packed_only else w.contiguous()
+        self.dtype, self.device = w.dtype, w.device
+
+    def nbytes(self):
+        return sum(t.numel() * t.element_size() for t in (self.packed, self.w) if t is not None)
+
+    def matmul(self, x):
+        """Library GEMM over many rows (prefill)."""
+        assert self.groups == 1 and x.dtype == self.dtype
+        return F.linear(x, self.w)
+
+
+def _gemm(wt, x, x_mode, epi, rows, **kw):
+    a = hip.TflGemm()
+    a.wp, a.x = wt.packed.data_ptr(), x.data_ptr()
+    a.rows, a.n, a.k, a.groups = rows, wt.n, wt.k, wt.groups
+    for name, v in kw.items():
+        setattr(a, name, v.data_ptr() if isinstance(v, torch.Tensor) else v)
+    hip.check(hip.latent_lib().tfl_gemm(ctypes.byref(a), _CODE[wt.dtype], hip.TFL_X[x_mode], hip.TFL_EPI[epi], _stream()), "tfl_gemm " + epi)
+
+
+def linear_f32(x, wt, n_real, out=None):
+    """fp32 x . W^T (logits, the token-side projection): x [rows, k] of the weight's type."""
+    _need(x)
+    rows = x.shape[0]
+    assert x.dtype == wt.dtype and x.shape[1] == wt.k
+    if out is None:
+        out = torch.empty(rows, n_real, dtype=torch.float32, device=x.device)
+    assert out.dtype == torch.float32 and out.shape[0] == rows and out.shape[1] >= n_real and out.stride(1) == 1
+    _gemm(wt, x, "t", "f32", rows, ld_x=x.stride(0), out_f=out, ld_f=out.stride(0), n_real=n_real)
+    return out
+
+
+def input_projection(h, wt, n_raw, act, act_off):
+    """All projections of the layer's one norm.  Returns (raw fp32 [rows, n_raw], per-panel sums of squares); gelu of the other
+    outputs goes to act[:, act_off:]."""
+    _need(h, act)
+    rows = h.shape[0]
+    assert h.dtype == wt.dtype == act.dtype and h.shape[1] == wt.k and act.shape[1] >= act_off + wt.n - n_raw
+    raw = torch.empty(rows, n_raw, dtype=torch.float32, device=h.device)
+    ss = torch.empty(rows, n_raw // 16, dtype=torch.float32, device=h.device)
+    tail = act[:, act_off:] if wt.n > n_raw else act
+    _gemm(wt, h, "t", "in", rows, ld_x=h.stride(0), out_f=raw, ld_f=n_raw, ss_out=ss, ss_ld=n_raw // 16, n_raw=n_raw,
+          out_t=tail, ld_t=act.stride(0))
+    return raw, ss
+
+
+def query_and_append(raw, ss, wt, g, q_norm, kv_norm, eps, rope, pos, slot, cache):
+    """Second stage of a decode step: raw's query latent normalised and up-projected (returned as unrotated [rows, H, N] and
+    [rows, H, C + R] with the rotated part filled in), raw's key latent normalised / rotated into the cache rows ``slot``.
+    g: LatentGeom."""
+    _need(raw, ss, cache, pos, slot)
+    _i32(pos, slot)
+    _f32(raw, ss, q_norm, kv_norm)
+    rows = raw.shape[0]
+    assert wt.n == g.H * (g.N + g.R) and wt.k == g.Q and cache.dtype == wt.dtype and cache.shape[1] == g.C + g.R and cache.is_contiguous()
+    assert pos.numel() == rows and slot.numel() == rows and raw.stride(0) == raw.shape[1] >= g.Q + g.C + g.R
+    qn = torch.empty(rows, g.H, g.N, dtype=wt.dtype, device=raw.device)
+    q = torch.empty(rows, g.H, g.C + g.R, dtype=wt.dtype, device=raw.device)
+    kv = raw[:, g.Q:]
+    _gemm(wt, raw, "f32_norm", "query", rows, ld_x=raw.stride(0), norm_w=q_norm, ss_in=ss, ss_n=g.Q // 16, ss_ld=ss.shape[1],
+          k_real=g.q_real, eps=eps, out_t=q, out_t2=qn, pos=pos, cos=rope.cos, sin=rope.sin, half=rope.half, max_pos=rope.max_pos,
+          H=g.H, N=g.N, R=g.R, C=g.C, c_real=g.c_real, kv_raw=kv, ld_kv=raw.stride(0), kv_norm_w=kv_norm, cache=cache,
+          cache_rows=cache.shape[0], slot=slot)
+    return qn, q
+
+
+def query_to_latent(qn, wt, q, g):
+    """q[:, h, :C] = qn[:, h] . Wuk_h (wt: groups of [C, N])."""
+    _need(qn, q)
+    rows = qn.shape[0]
+    assert (wt.groups, wt.n, wt.k) == (g.H, g.C, g.N) and qn.dtype == q.dtype == wt.dtype
+    _gemm(wt, qn, "t", "latent", rows, ld_x=g.H * g.N, x_group=g.N, out_t=q, H=g.H, C=g.C, R=g.R)
+    return q
+
+
+def latent_to_value(ol, wt, raw, gate_off, act, g):
+    """act[:, h*V:(h+1)*V] = (ol[:, h] . Wuv_h^T) * sigmoid(gate)."""
+    _need(ol, raw, act)
+    rows = ol.shape[0]
+    assert (wt.groups, wt.n, wt.k) == (g.H, g.V, g.C) and ol.dtype == act.dtype == wt.dtype and act.shape[1] >= g.H * g.V
+    assert raw.shape[1] >= gate_off + g.H * g.V
+    _gemm(wt, ol, "t", "gated", rows, ld_x=g.H * g.C, x_group=g.C, gate=raw[:, gate_off:], ld_gate=raw.stride(0), out_t=act,
+          ld_t=act.stride(0))
+
+
+def add_linear(act, wt, x):
+    """x (fp32) += act . W^T."""
+    _need(act, x)
+    _f32(x)
+    assert act.dtype == wt.dtype and act.shape[1] == wt.k and x.shape == (act.shape[0], wt.n) and x.is_contiguous()
+    _gemm(wt, act, "t", "residual", act.shape[0], ld_x=act.stride(0), out_f=x, ld_f=x.stride(0))
+
+
+def token_gate_linear(x, wt, table, ids, n_real):
+    """gelu(T(x) . W^T) * table[ids]: table is a column slice [vocab, n_real] of the token-side embedding."""
+    _need(x, table, ids)
+    _f32(x)
+    assert ids.dtype == torch.int64 and ids.numel() == x.shape[0] and table.dtype == wt.dtype and table.shape[1] == n_real
+    out = torch.empty(x.shape[0], wt.n, dtype=wt.dtype, device=x.device)
+    _gemm(wt, x, "f32", "token", x.shape[0], ld_x=x.stride(0), out_t=out, ld_t=wt.n, ids=ids, tok_table=table, ld_tok=table.stride(0),
+          vocab=table.shape[0], n_real=n_real)
+    return out
+
+
+def finish(x, norm_w, eps, width, dtype, embed=None, ids=None, y=None, y_w=None, step=None):
+    """Residual bookkeeping between two layers and the next norm; see tfl_finish.  x fp32 [rows, padded width] is updated in
+    place; returns h in ``dtype``."""
+    _need(x, norm_w, embed, ids, y, y_w, step)
+    _f32(x, norm_w, y_w, step)
+    rows, wp = x.shape
+    assert x.is_contiguous() and norm_w.numel() == wp and (step is None or step.numel() == wp)
+    assert embed is None or (embed.dtype == dtype and embed.shape[1] == wp and embed.is_contiguous() and ids.numel() == rows
+                             and ids.dtype == torch.int64)
+    assert y is None or (y.shape == (rows, wp) and y_w.numel() == wp and y.dtype in (dtype, torch.float32) and y.stride(1) == 1)
+    h = torch.empty(rows, wp, dtype=dtype, device=x.device)
+    hip.check(hip.latent_lib().tfl_finish(_p(embed), _p(ids), 0 if embed is None else embed.shape[0], _p(y),
+                                          int(y is not None and y.dtype == torch.float32), 0 if y is None else y.stride(0), _p(y_w),
+                                          _p(step), _p(norm_w), _p(x), _p(h), rows, wp, width, float(eps), _CODE[dtype], _stream()),
+              "tfl_finish")
+    return h
+
+
+def residual(d, x, want_copy):
+    """x += d; returns x in d's type when ``want_copy``."""
+    _need(d, x)
+    _f32(x)
+    assert d.shape == x.shape and d.is_contiguous() and x.is_contiguous()
+    xt = torch.empty_like(d) if want_copy else None
+    hip.check(hip.latent_lib().tfl_residual(_p(d), _p(x), _p(xt), d.numel(), _CODE[d.dtype], _stream()), "tfl_residual")
+    return xt
+
+
+def token_gate(s, table, ids, n_real):
+    _need(s, table, ids)
+    assert s.dtype == table.dtype and table.shape[1] == n_real and ids.dtype == torch.int64 and ids.numel() == s.shape[0]
+    out = torch.empty(s.shape[0], s.shape[1], dtype=s.dtype, device=s.device)
+    hip.check(hip.latent_lib().tfl_token_gate(_p(s), s.stride(0), _p(table), table.stride(0), _p(ids), table.shape[0], _p(out),
+                                              s.shape[0], s.shape[1], n_real, _CODE[s.dtype], _stream()), "tfl_token_gate")
+    return out
+
+
+def prepare(y, g, up_off, n_up, q_norm, kv_norm, eps, rope, pos, slot, cache, act, act_off, want_rows):
+    """Prefill half of the input projection (tfl_prepare): returns (cq, packed cache rows or None)."""
+    _need(y, pos, slot, cache, act)
+    _i32(pos, slot)
+    _f32(q_norm, kv_norm)
+    rows = y.shape[0]
+    assert y.stride(1) == 1 and pos.numel() == rows and slot.numel() == rows and cache.dtype == y.dtype == act.dtype
+    assert cache.shape[1] == g.C + g.R and cache.is_contiguous() and act.shape[1] >= act_off + n_up
+    cq = torch.empty(rows, g.Q, dtype=y.dtype, device=y.device)
+    ck = torch.empty(rows, g.C + g.R, dtype=y.dtype, device=y.device) if want_rows else None
+    hip.check(hip.latent_lib().tfl_prepare(_p(y), y.stride(0), g.Q, g.q_real, g.C, g.c_real, g.R, up_off, n_up, _p(q_norm), _p(kv_norm),
+                                           float(eps), _p(rope.cos), _p(rope.sin), rope.half, rope.max_pos, _p(pos), _p(slot),
+                                           _p(cache), cache.shape[0], _p(cq), _p(ck), _p(act[:, act_off:]) if n_up else None,
+                                           act.stride(0), rows, _CODE[y.dtype], _stream()), "tfl_prepare")
+    return cq, ck
+
+
+def gather_rows(cache, src):
+    _need(cache, src)
+    _i32(src)
+    out = torch.empty(src.numel(), cache.shape[1], dtype=cache.dtype, device=cache.device)
+    hip.check(hip.latent_lib().tfl_gather_rows(_p(cache), cache.shape[0], _p(src), _p(out), src.numel(), cache.shape[1],
+                                               _CODE[cache.dtype], _stream()), "tfl_gather_rows")
+    return out
+
+
+def attn_prefill(q, kv, ck, seq, max_new, pos, rope, gate, out, g, scale):
+    """q [tq, H*(N+R)], kv [tk, H*(N+V)], ck [tk, C+R], seq int32 [nseq, 4], gate / out [tq, >= H*V] views."""
+    _need(q, kv, ck, seq, pos, gate, out)
+    _i32(seq, pos)
+    tq, tk = q.shape[0], kv.shape[0]
+    assert q.dtype == kv.dtype == ck.dtype == gate.dtype == out.dtype and q.is_contiguous() and kv.is_contiguous() and ck.is_contiguous()
+    assert q.shape[1] == g.H * (g.N + g.R) and kv.shape[1] == g.H * (g.N + g.V) and ck.shape == (tk, g.C + g.R)
+    assert pos.numel() == tq and gate.shape[0] == tq and out.shape[0] == tq and seq.shape[1] == 4 and seq.is_contiguous()
+    assert gate.shape[1] >= g.H * g.V and out.shape[1] >= g.H * g.V
+    hip.check(hip.latent_lib().tfl_attn_prefill(_p(q), _p(kv), _p(ck), _p(seq), seq.shape[0], int(max_new), _p(pos), _p(rope.cos),
+                                                _p(rope.sin), rope.half, rope.max_pos, _p(gate), gate.stride(0), _p(out), out.stride(0),
+                                                tq, tk, g.H, g.N, g.R, g.V, g.C, float(scale), _CODE[q.dtype], _stream()),
+              "tfl_attn_prefill")
+
+
+def attn_decode(q, cache, table, klen, g, scale, max_len, nsplit=None):
+    """q [rows, H, C+R] against the paged cache -> [rows, H, C].  max_len sizes the split (klen is on the device)."""
+    _need(q, cache, table, klen)
+    _i32(table, klen)
+    rows = q.shape[0]
+    assert q.dtype == cache.dtype and q.is_contiguous() and q.shape[1:] == (g.H, g.C + g.R) and cache.shape[1] == g.C + g.R
+    assert cache.is_contiguous() and cache.shape[0] % PAGE == 0 and table.shape[0] == rows and table.stride(1) == 1 and klen.numel() == rows
+    L = hip.latent_lib()
+    if nsplit is None:
+        nsplit = L.tfl_attn_decode_pick_nsplit(rows, g.H, int(max_len))
+    n_ws = L.tfl_attn_decode_ws_floats(rows, g.H, g.C, nsplit)
+    ws = torch.empty(n_ws, dtype=torch.float32, device=q.device) if n_ws else None
+    out = torch.empty(rows, g.H, g.C, dtype=q.dtype, device=q.device)
+    hip.check(L.tfl_attn_decode(_p(q), _p(cache), cache.shape[0] // PAGE, _p(table), table.stride(0), _p(klen), _p(out), _p(ws), n_ws,
+                                rows, g.H, g.C, g.R, float(scale), nsplit, _CODE[q.dtype], _stream()), "tfl_attn_decode")
+    return out
+
+
+def decode_prep(lens, table, pos, slot, klen):
+    _need(lens, table, pos, slot, klen)
+    _i32(lens, table, pos, slot, klen)
+    rows = lens.numel()
+    assert table.shape[0] == rows and pos.numel() == rows and slot.numel() == rows and klen.numel() == rows
+    hip.check(hip.latent_lib().tfl_decode_prep(_p(lens), _p(table), table.stride(0), table.shape[1], _p(pos), _p(slot), _p(klen), rows,
+                                               _stream()), "tfl_decode_prep")

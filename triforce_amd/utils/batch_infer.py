@@ -1,0 +1,153 @@
+"""Engine for targets that are served autoregressively in batches (models with ``forward_batch``): prompts are prefilled
+together as one packed batch, then the sequences advance in lockstep, one token each, through one captured hipGraph per batch
+size.  It has the surface the decode loops drive (``engine``, ``inference``, ``decode_step``, ``clear_kv``) plus ``step`` for
+batches of named sequences."""
+import os
+
+import torch
+
+from .. import ops_latent as ol
+from ..models.cache import LatentBatch
+from . import graph_infer
+
+
+class _DecodeBuffers:
+    """Static device inputs of the decode step of B sequences.  ``lens`` advances on the device (ops_latent.decode_prep is part of
+    the step); the host uploads lengths and page tables only when the set of sequences or their pages changed."""
+
+    def __init__(self, cache, B):
+        dev = cache.device
+        self.B = B
+        self.ids = torch.zeros(B, dtype=torch.int64, device=dev)
+        self.lens = torch.full((B,), -1, dtype=torch.int32, device=dev)             # -1: idle row
+        self.table = torch.zeros(B, cache.columns, dtype=torch.int32, device=dev)
+        self.pos, self.slot, self.klen = (torch.zeros(B, dtype=torch.int32, device=dev) for _ in range(3))
+        self.batch = LatentBatch(True, self.pos, self.slot, table=self.table, klen=self.klen, max_len=cache.max_budget)
+        self.current = None                                     # (sequences, cache generation, lengths) the device holds
+
+
+class _DecodeStep:
+    """The lockstep decode forward of B sequences: eager, or captured once and replayed."""
+
+    def __init__(self, model, cache, B, use_graph):
+        self.model, self.cache, self.buf = model, cache, _DecodeBuffers(cache, B)
+        self.graph = self.logits = None
+        if use_graph:                                           # warm-up and capture run on idle rows: nothing is stored
+            self.graph, self.logits = graph_infer._capture(self._run, (), None, 2)
+
+    def _run(self):
+        b = self.buf
+        ol.decode_prep(b.lens, b.table, b.pos, b.slot, b.klen)
+        return self.model.forward_batch(b.ids, b.batch, self.cache)
+
+    def __call__(self, seqs, ids):
+        """seqs: the B sequences in order; ids: their next tokens (B,), on the device or the host.  Returns logits (B, V), valid
+        until the next call."""
+        b, c = self.buf, self.cache
+        before = tuple(c.length[s] for s in seqs)
+        c.extend([(s, 1) for s in seqs])
+        if b.current != (tuple(seqs), c.generation, before):
+            lens, table = c.tables(seqs)
+            b.table.copy_(table)
+            b.lens.copy_(lens - 1)
+        b.current = (tuple(seqs), c.generation, tuple(n + 1 for n in before))
+        b.ids.copy_(ids)
+        if self.graph is None:
+            return self._run()
+        self.graph.replay()
+        return self.logits
+
+
+class BatchInferenceEngine:
+    def __init__(self, model, cache, use_graphs=None):
+        self.model, self.kv_cache = model.eval(), cache
+        self.engine = self                                      # (the decode loops reach model and cache through .engine)
+        self.use_graphs = os.environ.get("TRIFORCE_DECODE_GRAPH", "1") != "0" if use_graphs is None else bool(use_graphs)
+        self._steps = {}
+
+    def clear_kv(self):
+        self.kv_cache.reset()
+
+    # -- named sequences -------------------------------------------------------------------------------------------------
+    @torch.inference_mode()
+    def step(self, entries, end=()):
+        """entries: [(sequence, its next tokens (list of ids), wanted places among them)]; ``end``: sequences that are finished
+        after this step.  Returns fp32 logits of the wanted places in order (None when there are none).  A step in which every
+        entry brings one token to a sequence that has some is a decode step; all others run the prefill kernels, cut into forwards
+        of at most graph_infer.PREFILL_CHUNK tokens."""
+        c = self.kv_cache
+        names = [s for s, _, _ in entries]
+        if len(set(names)) != len(names):
+            raise ValueError("a sequence appears twice in one step")
+        for s, toks, want in entries:
+            if len(toks) == 0:
+                raise ValueError(f"sequence {s!r}: no tokens")
+            if any(not 0 <= w < len(toks) for w in want):
+                raise ValueError(f"sequence {s!r}: a wanted place is outside its tokens")
+            if any(not 0 <= t < self.model.vocab_size for t in toks):
+                raise ValueError(f"sequence {s!r}: a token id is outside the vocabulary")
+        for s in end:
+            if s not in c.length and s not in names:
+                raise KeyError(f"unknown sequence {s!r}")
+        out = None
+        if entries:
+            if all(len(toks) == 1 and c.length.get(s, 0) > 0 for s, toks, _ in entries):
+                logits = self.decode(names, torch.tensor([toks[0] for _, toks, _ in entries], dtype=torch.int64))
+                rows = [b for b, (_, _, want) in enumerate(entries) for _ in want]
+                if rows:
+                    out = logits[rows] if rows != list(range(len(entries))) else logits.clone()
+            else:
+                out = self._prefill(entries)
+        for s in end:
+            c.release(s)
+        return out
+
+    def _prefill(self, entries):
+        c = self.kv_cache
+        if c.tokens + sum(len(t) for _, t, _ in entries) > c.max_budget:
+            raise IndexError(f"LatentCache overflow: {c.tokens} + {sum(len(t) for _, t, _ in entries)} > {c.max_budget} tokens")
+        at = [0] * len(entries)
+        rows = {}                                               # (entry, place) -> logits row
+        while True:
+            room, portion = graph_infer.PREFILL_CHUNK, []
+            for e, (s, toks, want) in enumerate(entries):
+                n = min(room, len(toks) - at[e])
+                if n > 0:
+                    portion.append((e, at[e], n))
+                    room -= n
+            if not portion:
+                break
+            ids, plan, keys = [], [], []
+            for e, a, n in portion:
+                s, toks, want = entries[e]
+                places = sorted({w for w in want if a <= w < a + n})
+                ids += list(toks[a:a + n])
+                plan.append((s, n, [w - a for w in places]))
+                keys += [(e, w) for w in places]
+                at[e] = a + n
+            batch = c.plan_prefill(plan)
+            logits = self.model.forward_batch(torch.tensor(ids, dtype=torch.int64).to(c.device), batch, c)
+            if keys:
+                rows.update({k: logits[j] for j, k in enumerate(keys)})
+        out = [rows[(e, w)] for e, (_, _, want) in enumerate(entries) for w in want]
+        return torch.stack(out) if out else None
+
+    @torch.inference_mode()
+    def decode(self, seqs, ids):
+        """One token each for ``seqs``: logits (B, V), valid until the next step of that batch size."""
+        B = len(seqs)
+        st = self._steps.get(B)
+        if st is None:
+            st = self._steps[B] = _DecodeStep(self.model, self.kv_cache, B, self.use_graphs)
+        return st(seqs, ids.reshape(-1))
+
+    # -- the single-sequence surface of utils/decoding.py ----------------------------------------------------------------
+    @torch.inference_mode()
+    def inference(self, input_ids, **_):
+        """Prompt (or a further portion) of the cache's default sequence -> logits (1, rows, V) like the other engines."""
+        return graph_infer.chunked_prefill(lambda ids, last_rows=None: self.model.forward(ids, self.kv_cache, last_rows=last_rows).logits,
+                                           input_ids)
+
+    @torch.inference_mode()
+    def decode_step(self, input_ids):
+        return self.decode([self.kv_cache.DEFAULT], input_ids).unsqueeze(0)

@@ -71,6 +71,65 @@ def Autoregressive(tokenizer, graph_engine, input_ids, max_len=256, top_k=-1, to
     return n / (time2 - time1)
 
 
+@torch.inference_mode()
+def AutoregressiveBatch(tokenizer, graph_engine, prompts, max_len=256, top_k=-1, top_p=0.9, temperature=0.6, verbose=False, rng=None,
+                        return_tokens=False):
+    """``Autoregressive`` for many prompts on an engine with named sequences (utils/batch_infer.py).  ``prompts``: list of token
+    id lists or (1, n) tensors of any lengths; ``max_len``: tokens to generate behind the first sampled one, an int or one per
+    prompt.  Prompts are taken in order, as many at a time as the cache has sequences and tokens for; such a batch is prefilled
+    together and decoded in lockstep, its shorter requests leave early and give their pages back.  Returns tokens / s over the
+    decode steps [, the token lists]."""
+    eng = graph_engine.engine
+    cache, device = eng.kv_cache, eng.model.device
+    rng = rng or UniformSource(device)
+    prompts = [p.reshape(-1).tolist() if torch.is_tensor(p) else list(p) for p in prompts]
+    lens = [max_len] * len(prompts) if isinstance(max_len, int) else list(max_len)
+    assert len(lens) == len(prompts)
+    sampling = dict(temperature=temperature, top_k=top_k, top_p=top_p)
+
+    def draw(logits):                                # (rows, V) -> (rows,) ids; rows take their uniforms in order
+        probs = norm_logits(logits, **sampling)
+        return torch.cat([sample(row, rng=rng).view(1) for row in probs])
+    out, spent, made, nxt = {}, 0.0, 0, 0
+    while nxt < len(prompts):
+        cache.reset()
+        group, tokens = [], 0
+        while nxt < len(prompts) and len(group) < cache.max_batch and tokens + len(prompts[nxt]) + lens[nxt] <= cache.max_budget:
+            tokens += len(prompts[nxt]) + lens[nxt]
+            group.append(nxt)
+            nxt += 1
+        if not group:
+            raise IndexError(f"prompt {nxt} does not fit the cache: {len(prompts[nxt])} + {lens[nxt]} > {cache.max_budget} tokens")
+        ids = draw(graph_engine.step([(i, prompts[i], [len(prompts[i]) - 1]) for i in group]))
+        live, steps = list(group), [(list(group), ids)]
+        _sync(device)
+        t0 = time.time()
+        for n in range(max(lens[i] for i in group)):    # no host sync inside the loop
+            keep = [b for b, i in enumerate(live) if lens[i] > n]
+            for b, i in enumerate(live):
+                if lens[i] <= n:
+                    cache.release(i)
+            if len(keep) < len(live):
+                ids, live = ids[keep], [live[b] for b in keep]
+            ids = draw(graph_engine.decode(live, ids))
+            steps.append((list(live), ids))
+            made += len(live)
+        _sync(device)
+        spent += time.time() - t0
+        for who, row in steps:
+            for i, t in zip(who, row.tolist()):
+                out.setdefault(i, []).append(t)
+        for i in live:
+            cache.release(i)
+    if verbose:
+        for i in range(len(prompts)):
+            for t in out[i]:
+                spec_stream(t, tokenizer, "cyan")
+            print()
+    speed = made / spent if spent else 0.0
+    return (speed, [out[i] for i in range(len(prompts))]) if return_tokens else speed
+
+
 # The host waits for a decision record by polling pinned memory.  A poll loop that never yields can sit on the core a HIP
 # runtime thread needs (launch hand-off, completion signals): measured on 8-vCPU boxes, the hop between an accept kernel
 # and the next launch was 12 us in one process and 61 us in another for the same code (profiles/r04_host_path_ab.txt).

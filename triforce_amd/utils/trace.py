@@ -1,0 +1,54 @@
+"""Replay of a token trace: given ids go through a model step by step and the wanted logits are written to files; nothing is
+sampled.  Command line: bin/trace_run.  The steps run on the engine, cache and kernels that generation uses."""
+import argparse
+import json
+import os
+import sys
+
+import torch
+
+
+def parse(argv=None):
+    ap = argparse.ArgumentParser(description="run given tokens through a model step by step and write logits; steps are JSON lines "
+                                             "on standard input: {\"step\": n, \"entries\": [{\"id\", \"tokens\", \"want\"}], \"end\": [ids]}")
+    ap.add_argument("--model", required=True, help="checkpoint directory (config.json, *.safetensors)")
+    ap.add_argument("--dtype", default="bfloat16", choices=["bfloat16", "float32"])
+    ap.add_argument("--out", required=True, help="directory for <step>.f32 files (little-endian fp32, [wanted, vocabulary])")
+    ap.add_argument("--max-tokens", type=int, required=True, help="most tokens that live requests hold at any time")
+    ap.add_argument("--max-batch", type=int, default=256, help="most live requests")
+    ap.add_argument("--device", default="cuda:0")
+    return ap.parse_args(argv)
+
+
+def make_engine(args):
+    from ..models import registry
+    from ..models.cache import LatentCache
+    from .batch_infer import BatchInferenceEngine
+    cls = registry.model_class(registry.architecture_of(args.model))
+    if not hasattr(cls, "forward_batch"):
+        raise NotImplementedError(f"{cls.__name__} is not served in batches")
+    model = registry.load_model(args.model, args.device, torch_dtype=getattr(torch, args.dtype))
+    return BatchInferenceEngine(model, LatentCache(model, max_budget=args.max_tokens, max_batch=min(args.max_batch, args.max_tokens)))
+
+
+def replay(engine, lines, out_dir, report=print):
+    """lines: iterable of JSON step lines.  ``report`` is called with "done <step>" after each of them."""
+    for line in lines:
+        if not line.strip():
+            continue
+        s = json.loads(line)
+        logits = engine.step([(e["id"], e["tokens"], e.get("want", [])) for e in s["entries"]], s.get("end", []))
+        if logits is not None:
+            path = os.path.join(out_dir, f"{s['step']}.f32")
+            with open(path + ".part", "wb") as f:
+                f.write(logits.to(torch.float32).cpu().numpy().astype("<f4").tobytes())
+            os.replace(path + ".part", path)
+        report(f"done {s['step']}")
+
+
+def main(argv=None):
+    args = parse(argv)
+    torch.backends.cuda.matmul.allow_tf32 = False               # float32 means float32
+    engine = make_engine(args)
+    replay(engine, sys.stdin, args.out, lambda text: print(text, flush=True))
+    return 0

@@ -3,6 +3,9 @@
 TEST INFRASTRUCTURE ONLY: the checker of tests/test_latent_*.py; the product (triforce_amd/) never imports it and it imports
 nothing from the product.  Everything runs in the dtype of the weights it is given (float32 or float64).
 
+``operand`` (everywhere): what happens to an activation right before a matrix product - nothing, or a rounding, which tells how
+far a product in a shorter format may move the result.
+
 Notation: T tokens, d = width, H heads, N / R = unrotated / rotated query-key size of a head, V = value size, C = latent size.
 """
 import math
@@ -12,6 +15,10 @@ import torch
 
 def gelu(z):
     return 0.5 * z * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z ** 3)))
+
+
+def exact(x):
+    return x
 
 
 def rms(x, eps):
@@ -53,33 +60,35 @@ def rotate(x, positions, rot):
     return y
 
 
-def latent_attention(h, w, mixer, eps, positions=None):
+def latent_attention(h, w, mixer, eps, positions=None, operand=exact):
     """w: the mixer's tensors by short name ("dq", "dq.norm", "uq", "dkv", "dkv.norm", "uk", "uv", "g", "o")."""
     T = h.shape[0]
     H, N, R, V, C = mixer["heads"], mixer["dim"], mixer["rot_dim"], mixer["vdim"], mixer["kv_rank"]
     pos = torch.arange(T) if positions is None else positions
-    q = (rms(h @ w["dq"].T, eps) * w["dq.norm"]) @ w["uq"].T
+    h = operand(h)
+    q = operand(rms(h @ w["dq"].T, eps) * w["dq.norm"]) @ w["uq"].T
     q = q.view(T, H, N + R)
     qn, qr = q[..., :N], rotate(q[..., N:], pos, mixer["rot"])
     kv = h @ w["dkv"].T
-    c = rms(kv[:, :C], eps) * w["dkv.norm"]
+    c = operand(rms(kv[:, :C], eps) * w["dkv.norm"])
     kr = rotate(kv[:, C:], pos, mixer["rot"])
     kn = (c @ w["uk"].T).view(T, H, N)
     v = (c @ w["uv"].T).view(T, H, V)
+    qn, kn, qr, kr, v = (operand(x) for x in (qn, kn, qr, kr, v))
     s = torch.einsum("thn,shn->hts", qn, kn) + torch.einsum("thr,sr->hts", qr, kr)
     s = s * mixer["scale"]
     s = s.masked_fill(pos[None, None, :] > pos[None, :, None], float("-inf"))
     o = torch.einsum("hts,shv->thv", torch.softmax(s, dim=-1), v).reshape(T, H * V)
-    return (o * torch.sigmoid(h @ w["g"].T)) @ w["o"].T
+    return operand(o * torch.sigmoid(h @ w["g"].T)) @ w["o"].T
 
 
-def feed_forward(h, w):
-    return gelu(h @ w["up"].T) @ w["down"].T
+def feed_forward(h, w, operand=exact):
+    return operand(gelu(operand(h) @ w["up"].T)) @ w["down"].T
 
 
-def token_side(x, e, w, eps):
+def token_side(x, e, w, eps, operand=exact):
     """Per-layer token input: w has "gate", "proj", "norm"; e is the layer's part of the token's side embedding."""
-    y = (gelu(x @ w["gate"].T) * e) @ w["proj"].T
+    y = operand(gelu(operand(x) @ w["gate"].T) * e) @ w["proj"].T
     return rms(y, eps) * w["norm"]
 
 
@@ -99,7 +108,7 @@ def _under(sd, prefix):
     return {k[len(prefix):]: v for k, v in sd.items() if k.startswith(prefix)}
 
 
-def forward(cfg, sd, tokens, trace=None):
+def forward(cfg, sd, tokens, trace=None, operand=exact):
     """tokens: list of ids -> (T, vocab) logits.  ``trace``: list that receives the residual stream after every layer run."""
     ids = torch.as_tensor(tokens, dtype=torch.long)
     eps = cfg["norm"]["eps"]
@@ -109,13 +118,13 @@ def forward(cfg, sd, tokens, trace=None):
         if first:
             x = x + sd["loop.step"][t]
         h = rms(x, eps) * sd[f"l{i}.norm1"]
-        d = latent_attention(h, _under(sd, f"l{i}.mix."), L["mixer"], eps)
+        d = latent_attention(h, _under(sd, f"l{i}.mix."), L["mixer"], eps, operand=operand)
         if L.get("mlp") is not None:
-            d = d + feed_forward(h, _under(sd, f"l{i}.mlp."))
+            d = d + feed_forward(h, _under(sd, f"l{i}.mlp."), operand)
         x = x + d
         if cfg.get("token_side") is not None:
             n = cfg["token_side"]["dim"]
-            x = x + token_side(x, sd["side.embed"][ids][:, i * n:(i + 1) * n], _under(sd, f"l{i}.side."), eps)
+            x = x + token_side(x, sd["side.embed"][ids][:, i * n:(i + 1) * n], _under(sd, f"l{i}.side."), eps, operand)
         if trace is not None:
             trace.append(x)
-    return (rms(x, eps) * sd["final.norm"]) @ sd["embed"].T
+    return operand(rms(x, eps) * sd["final.norm"]) @ sd["embed"].T

@@ -1,0 +1,287 @@
+"""Befidra without a GPU: configuration, registry, checkpoint names, cache manager, command lines, and the oracle's own
+sensitivity to every mechanism (a test that cannot see a fault proves nothing)."""
+import copy
+import ctypes
+import json
+import math
+import os
+import re
+
+import pytest
+import torch
+
+from oracle import ref_latent as R
+from tests import latent_helpers as H
+from triforce_amd.models import registry, zoo
+from triforce_amd.models.cache import LatentCache
+from triforce_amd.models.config_befidra import BefidraConfig
+from triforce_amd.models.latent_core import LatentWeights, RotaryTable, rotary_frequencies
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+
+# ---- library --------------------------------------------------------------------------------------------------------------
+def test_latent_library_exports_what_the_header_declares():
+    from triforce_amd import hip
+    src = re.sub(r"/\*.*?\*/", "", open(os.path.join(ROOT, "include", "triforce_latent.h")).read(), flags=re.S)
+    names = set(re.findall(r"\b(tfl_[a-z0-9_]+)\s*\(", src))
+    assert names == set(hip.LATENT_SIGNATURES)
+    lib = hip.latent_lib()
+    assert all(hasattr(lib, n) for n in names)
+
+
+def test_gemm_structure_matches_the_header():
+    from triforce_amd import hip
+    src = open(os.path.join(ROOT, "include", "triforce_latent.h")).read()
+    body = re.sub(r"/\*.*?\*/", "", re.search(r"typedef struct TflGemm \{(.*?)\} TflGemm;", src, re.S).group(1), flags=re.S)
+    fields = []
+    for decl in body.split(";"):
+        decl = re.sub(r"^(const )?(void|float|int64_t|int32_t)\s*", "", decl.strip())
+        fields += [f.strip().lstrip("*").strip() for f in decl.split(",") if f.strip()]
+    assert fields == [n for n, _ in hip.TflGemm._fields_]
+
+
+def test_bad_arguments_are_refused_before_any_launch():
+    from triforce_amd import hip
+    L = hip.latent_lib()
+    a = hip.TflGemm()
+    assert L.tfl_gemm(ctypes.byref(a), 0, 0, 0, None) == -22
+    a.wp = a.x = a.out_f = 1 << 20
+    a.rows, a.n, a.k, a.groups, a.n_real, a.ld_f, a.ld_x = 1, 16, 32, 1, 16, 16, 32
+    a.k = 40
+    assert L.tfl_gemm(ctypes.byref(a), 0, 0, 0, None) == -22
+    assert L.tfl_attn_decode(1, 1, 1, 1, 1, 1, 1, None, 0, 1, 1, 48, 32, 1.0, 1, 0, None) == -22        # latent not padded
+    assert L.tfl_attn_decode(1, 1, 1, 1, 1, 1, 1, None, 0, 1, 1, 64, 32, 1.0, 4, 0, None) == -28        # no workspace
+    for rows in (1, 3, 64):
+        for heads in (1, 16, 33, 128):
+            for n in (1, 64, 5000, 131072):
+                s = L.tfl_attn_decode_pick_nsplit(rows, heads, n)
+                assert 1 <= s <= 256 and (s == 1 or s <= math.ceil(n / 128))
+
+
+# ---- configuration and registry -------------------------------------------------------------------------------------------
+@pytest.mark.parametrize("name", sorted(H.CONFIGS))
+def test_config_round_trip_and_layer_order(name):
+    d = H.CONFIGS[name]
+    c = registry.config_from_dict(d)
+    assert isinstance(c, BefidraConfig)
+    assert BefidraConfig.from_dict(c.to_dict()).to_dict() == c.to_dict()
+    assert [(i, t or 0, f) for i, t, f in c.layer_runs()] == R.layer_runs(d)
+
+
+def test_layer_runs_of_a_loop():
+    c = registry.config_from_dict(H.CONFIGS["mixed"])
+    assert [(i, t, f) for i, t, f in c.layer_runs()] == \
+        [(0, None, False), (1, 0, True), (2, 0, False), (1, 1, True), (2, 1, False), (1, 2, True), (2, 2, False)]
+
+
+@pytest.mark.parametrize("change, message", [
+    (lambda d: d["layers"][0].update(type="other"), "mixer type"), (lambda d: d["layers"][0]["mlp"].update(kind="gated"), "feed-forward"),
+    (lambda d: d.update(loop=dict(start=1, stop=9, times=1)), "loop"), (lambda d: d["layers"][0]["mixer"]["rot"].update(dims=3), "even"),
+    (lambda d: d["layers"][0]["mixer"]["rot"]["scaling"].pop("fast"), "fast"), (lambda d: d["layers"][0]["mixer"].update(heads=0), "heads")])
+def test_config_refuses_what_it_does_not_know(change, message):
+    d = copy.deepcopy(H.CONFIGS["mixed"])
+    change(d)
+    with pytest.raises(ValueError, match=message):
+        BefidraConfig.from_dict(d)
+
+
+def test_registry_chooses_by_config(tmp_path):
+    assert registry.architecture_of({"architectures": ["LlamaForCausalLM"]}) == "LlamaForCausalLM"
+    assert registry.architecture_of({}) == "LlamaForCausalLM"
+    with pytest.raises(NotImplementedError):
+        registry.architecture_of({"architecture": "Nobody"})
+    (tmp_path / "config.json").write_text(json.dumps(H.CONFIGS["plain"]))
+    assert registry.model_class(registry.architecture_of(str(tmp_path))).__name__ == "BefidraForCausalLM"
+    assert type(zoo.config("befidra-7B")).__name__ == "BefidraConfig" and type(zoo.config("llama-68M")).__name__ == "LlamaConfig"
+
+
+def test_speculative_scripts_refuse_and_generate_parses():
+    from triforce_amd.models.modeling_llama import LlamaForCausalLM
+    from triforce_amd.utils import cli
+    with pytest.raises(NotImplementedError, match="generate"):
+        cli.load_causal_lm(LlamaForCausalLM, "random:1", "befidra-tiny", "cpu")
+    a = cli.parse("generate", ["--greedy", "--batch", "3"])
+    assert (a.temp, a.top_p, a.batch, a.target) == (1.0, 1e-9, 3, "befidra-tiny")
+
+
+def test_weights_name_missing_and_misshapen_tensors():
+    d = H.CONFIGS["plain"]
+    sd = H.weights(d, 1)
+    W = LatentWeights(BefidraConfig.from_dict(d), "cpu", torch.float32)
+    with pytest.raises(KeyError, match="l0.mix.g"):
+        W.load_state_dict({k: v for k, v in sd.items() if k != "l0.mix.g"})
+    sd["l1.mix.uv"] = sd["l1.mix.uv"][:-1]
+    with pytest.raises(ValueError, match="l1.mix.uv"):
+        W.load_state_dict(sd)
+
+
+def test_packed_tiles_hold_the_matrix():
+    from triforce_amd.ops_latent import pack_tiles
+    w = torch.arange(48 * 64).float().view(48, 64)
+    p = pack_tiles(w)
+    for n, k in ((0, 0), (17, 33), (47, 63), (30, 8)):
+        assert p[n // 16, k // 32, (k % 32) // 8, n % 16, k % 8] == w[n, k]
+
+
+@pytest.mark.parametrize("rot", [dict(dims=16, base=10000.0), dict(dims=16, base=500.0, scaling=dict(factor=4.0, original=64, fast=8.0, slow=1.0)),
+                                 dict(dims=2, base=100.0, scaling=dict(factor=2.0, original=32, fast=1.0, slow=1.0))])
+def test_rotary_tables_against_the_oracle(rot):
+    from triforce_amd.models.config_befidra import RotarySpec
+    spec = RotarySpec(**rot)
+    f, m = rotary_frequencies(spec)
+    fo, mo = R.frequencies(rot)
+    assert f == pytest.approx(fo, rel=1e-14) and m == pytest.approx(mo)
+    t = RotaryTable(spec, 700, "cpu")
+    x = torch.randn(700, rot["dims"])
+    y = R.rotate(x.double(), torch.arange(700), rot)
+    u, v = x[:, 0::2], x[:, 1::2]
+    assert torch.allclose(u * t.cos - v * t.sin, y[:, 0::2].float(), atol=1e-6)
+    assert torch.allclose(v * t.cos + u * t.sin, y[:, 1::2].float(), atol=1e-6)
+
+
+# ---- cache manager --------------------------------------------------------------------------------------------------------
+class _Model:
+    device, dtype = torch.device("cpu"), torch.float32
+    asked = 0
+
+    def cache_widths(self):
+        return [64, 96, 64]
+
+    def prepare_positions(self, n):
+        self.asked = n
+
+
+def test_cache_pages_grow_are_freed_and_used_again():
+    m = _Model()
+    c = LatentCache(m, max_budget=200, max_batch=3)
+    assert m.asked == 200 and c.n_pages == 4 + 2 and [r.shape for r in c.rows] == [(384, 64), (384, 96), (384, 64)]
+    c.extend([("a", 64), ("b", 1)])
+    assert len(c.pages["a"]) == 1 and len(c.pages["b"]) == 1
+    c.extend([("a", 1)])
+    assert len(c.pages["a"]) == 2
+    rows = c.cache_rows("a", 0, 65).tolist()
+    assert rows[:64] == [c.pages["a"][0] * 64 + j for j in range(64)] and rows[64] == c.pages["a"][1] * 64
+    assert c.cache_rows("a", 63, 2).tolist() == rows[63:65]
+    gone = set(c.pages["a"])
+    c.release("a")
+    c.extend([("c", 100)])
+    assert set(c.pages["c"]) == gone and c.tokens == 101
+    with pytest.raises(IndexError):
+        c.extend([("b", 100)])                                   # 201 tokens
+    assert c.tokens == 101 and c.length["b"] == 1, "a refused step changes nothing"
+    c.extend([("b", 1), ("d", 98)])                              # the whole budget, three part-filled pages
+    with pytest.raises(IndexError):
+        LatentCache(_Model(), 200, 1).extend([("a", 1), ("b", 1)])
+    c.reset()
+    assert c.tokens == 0 and len(c.free) == c.n_pages
+
+
+def test_cache_never_runs_out_of_pages_inside_its_budget():
+    g = torch.Generator().manual_seed(3)
+    for budget, batch in ((1, 1), (64, 64), (65, 5), (500, 70), (1000, 130)):
+        c = LatentCache(_Model(), budget, batch)
+        for _ in range(300):
+            if c.length and torch.rand(1, generator=g) < 0.1:
+                c.release(sorted(c.length)[int(torch.randint(len(c.length), (1,), generator=g))])
+            left = budget - c.tokens
+            if left == 0:
+                c.release(sorted(c.length)[0])
+                continue
+            n = min(left, int(torch.randint(1, 3 if batch > 50 else 70, (1,), generator=g)))
+            name = int(torch.randint(batch, (1,), generator=g))
+            c.extend([(name, n)])
+        owned = [p for ps in c.pages.values() for p in ps] + c.free
+        assert sorted(owned) == list(range(c.n_pages))
+
+
+def test_prefill_plan_positions_slots_and_keys():
+    c = LatentCache(_Model(), 400, 4)
+    b = c.plan_prefill([("a", 70, [69]), ("b", 3, range(3))])
+    assert not b.decode and b.key_rows is None and b.max_new == 70
+    assert b.pos.tolist() == list(range(70)) + [0, 1, 2] and b.seq.tolist() == [[0, 70, 0, 70], [70, 3, 70, 3]]
+    assert b.want.tolist() == [69, 70, 71, 72]
+    b = c.plan_prefill([("b", 2, []), ("a", 5, [0])])
+    assert b.pos.tolist() == [3, 4, 70, 71, 72, 73, 74] and b.seq.tolist() == [[0, 2, 0, 5], [2, 5, 5, 75]]
+    assert b.key_rows.tolist() == c.cache_rows("b", 0, 5).tolist() + c.cache_rows("a", 0, 75).tolist()
+    assert b.slot.tolist() == c.cache_rows("b", 3, 2).tolist() + c.cache_rows("a", 70, 5).tolist()
+    assert b.want.tolist() == [2]
+    lens, table = c.tables(["b", "a"])
+    assert lens.tolist() == [5, 75] and table[1, :2].tolist() == c.pages["a"]
+
+
+# ---- oracle ---------------------------------------------------------------------------------------------------------------
+def _twist(cfg, sd, what):
+    cfg, sd = copy.deepcopy(cfg), dict(sd)
+    if what == "one pass less":
+        cfg["loop"]["times"] -= 1
+    elif what == "no yarn":
+        cfg["layers"][0]["mixer"]["rot"]["scaling"] = None
+    elif what == "no step":
+        sd["loop.step"] = torch.zeros_like(sd["loop.step"])
+    elif what == "steps swapped":
+        sd["loop.step"] = sd["loop.step"].flip(0)
+    elif what == "no gate":
+        sd["l0.mix.g"] = torch.zeros_like(sd["l0.mix.g"])
+    elif what == "no feed-forward":
+        cfg["layers"][0]["mlp"] = None
+    elif what == "side part of the neighbour":
+        n = cfg["token_side"]["dim"]
+        sd["side.embed"] = sd["side.embed"].roll(n, dims=1)
+    elif what == "key rotation off by one":
+        sd["l2.mix.dkv"] = sd["l2.mix.dkv"].roll(1, dims=0)
+    elif what == "scale":
+        cfg["layers"][2]["mixer"]["scale"] *= 1.05
+    elif what == "eps":
+        cfg["norm"]["eps"] = 1e-6
+    elif what == "query norm":
+        sd["l0.mix.dq.norm"] = torch.ones_like(sd["l0.mix.dq.norm"])
+    return cfg, sd
+
+
+@pytest.mark.parametrize("what", ["one pass less", "no yarn", "no step", "steps swapped", "no gate", "no feed-forward",
+                                  "side part of the neighbour", "key rotation off by one", "scale", "eps", "query norm"])
+def test_a_fault_in_a_mechanism_shows(what):
+    """The fault is planted in the oracle; the bound is ten times what the fp32 device tests allow."""
+    cfg = H.CONFIGS["mixed"]
+    sd = H.weights(cfg, 5)
+    toks = H.tokens_of(cfg, 40, 6)
+    good = H.oracle_logits(cfg, sd, toks)
+    bad = H.oracle_logits(*_twist(cfg, sd, what), toks)
+    assert H.error(bad[20:], good[20:]) > 10 * 5e-5
+
+
+def test_oracle_is_causal_and_position_dependent():
+    cfg = H.CONFIGS["mixed"]
+    sd = H.weights(cfg, 7)
+    toks = H.tokens_of(cfg, 30, 8)
+    a = H.oracle_logits(cfg, sd, toks)
+    b = H.oracle_logits(cfg, sd, toks[:29] + [(toks[29] + 1) % cfg["vocab"]])
+    assert torch.equal(a[:29], b[:29]) and not torch.equal(a[29], b[29])
+    c = H.oracle_logits(cfg, sd, toks[1:])
+    assert H.error(c[5:], a[6:]) > 1e-2                        # (the first token is gone and every position moved)
+
+
+def test_trace_command_line():
+    from triforce_amd.utils import trace
+    a = trace.parse(["--model", "m", "--out", "o", "--max-tokens", "9", "--dtype", "float32"])
+    assert (a.model, a.out, a.max_tokens, a.dtype) == ("m", "o", 9, "float32")
+    with pytest.raises(SystemExit):
+        trace.parse(["--model", "m", "--out", "o", "--max-tokens", "9", "--dtype", "float16"])
+
+
+def test_trace_replay_protocol(tmp_path):
+    """Steps in order, a file only where something is wanted, a line after every step."""
+    from triforce_amd.utils import trace
+    calls, lines = [], []
+
+    class Engine:
+        def step(self, entries, end):
+            calls.append((entries, end))
+            n = sum(len(w) for _, _, w in entries)
+            return torch.arange(float(n * 4)).view(n, 4) if n else None
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": [1, 2], "want": [1]}], "end": []},
+             {"step": 1, "entries": [{"id": "a", "tokens": [3], "want": []}], "end": ["a"]}]
+    trace.replay(Engine(), [json.dumps(s) + "\n" for s in steps] + ["\n"], str(tmp_path), lines.append)
+    assert lines == ["done 0", "done 1"] and calls[1] == ([("a", [3], [])], ["a"])
+    assert (tmp_path / "0.f32").stat().st_size == 16 and not (tmp_path / "1.f32").exists()

@@ -61,9 +61,12 @@ class _DecodeStep:
 class BatchInferenceEngine:
     def __init__(self, model, cache, use_graphs=None):
         self.model, self.kv_cache = model.eval(), cache
-        self.engine = self                                      # (the decode loops reach model and cache through .engine)
         self.use_graphs = os.environ.get("TRIFORCE_DECODE_GRAPH", "1") != "0" if use_graphs is None else bool(use_graphs)
         self._steps = {}
+
+    @property
+    def engine(self):                                           # (the decode loops reach model and cache through .engine)
+        return self
 
     def clear_kv(self):
         self.kv_cache.reset()

@@ -1,0 +1,267 @@
+"""``python bench.py --design befidra``: throughput and per-kernel roofline distance of the latent-attention design beside the
+Llama of equal width, heads and feed-forward (the closest other model), on one GPU with random weights.
+
+One JSON line per measurement, one summary line at the end.  Kernel times come from a hipGraph of back-to-back calls that rotate
+over the layers' weights and caches (several times the Infinity Cache), so they are launch-free and cache-cold.  "of roofline" is
+the larger of bytes / 8 TB/s and flops / 2.5 PFLOP/s over the measured time.
+"""
+import json
+import time
+
+import torch
+
+HBM, MFMA = 8.0e12, 2.5e15
+LAYERS = 4                     # per model: enough to rotate over
+WIDTH, FF, HEADS = 4096, 11008, 32
+
+
+def _emit(row):
+    print(json.dumps(row), flush=True)
+
+
+def _graph_us(calls, reps=5, loops=3):
+    """Mean time of one call of ``calls`` (a list of closures) inside a captured graph of loops * len(calls) launches."""
+    from triforce_amd.utils import graph_infer
+    with torch.inference_mode():
+        graph, _ = graph_infer._capture(lambda: [c() for _ in range(loops) for c in calls][-1], (), None, 1)
+        graph.replay()
+        torch.cuda.synchronize()
+        a, b = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+        best = float("inf")
+        for _ in range(reps):
+            a.record()
+            graph.replay()
+            b.record()
+            b.synchronize()
+            best = min(best, a.elapsed_time(b))
+    return 1e3 * best / (loops * len(calls))
+
+
+def _kernel(rows, model, name, calls, nbytes, flops=0.0, like=None, **info):
+    us = _graph_us(calls)
+    ideal = 1e6 * max(nbytes / HBM, flops / MFMA)
+    row = dict(kind="kernel", model=model, kernel=name, rows=rows, us=round(us, 2), gbps=round(nbytes / us / 1e3, 1),
+               tflops=round(flops / us / 1e6, 1), of_roofline=round(ideal / us, 3), like=like, **info)
+    _emit(row)
+    return row
+
+
+def befidra_model(device):
+    from triforce_amd.models import zoo
+    from triforce_amd.models.modeling_befidra import BefidraForCausalLM
+    d = json.loads(json.dumps(zoo.CONFIGS["befidra-7B"]))
+    d["layers"], d["loop"] = d["layers"][:LAYERS], None
+    from triforce_amd.models import registry
+    return BefidraForCausalLM(registry.config_from_dict(d), device).init_random(1)
+
+
+def llama_model(device):
+    from triforce_amd.models.config_yarn import LlamaConfig
+    from triforce_amd.models.modeling_llama import LlamaForCausalLM
+    cfg = LlamaConfig(hidden_size=WIDTH, intermediate_size=FF, num_hidden_layers=LAYERS, num_attention_heads=HEADS,
+                      max_position_embeddings=131072)
+    return LlamaForCausalLM(cfg, device).init_random(1)
+
+
+# ---- decode kernels ---------------------------------------------------------------------------------------------------------
+def befidra_decode_kernels(m, rows, ctx):
+    from triforce_amd import ops_latent as ol
+    from triforce_amd.models.cache import LatentCache
+    W, dev = m.weights, m.device
+    g = W.layers[0].geom
+    cache = LatentCache(m, max_budget=rows * (ctx + 64), max_batch=rows)
+    for r in cache.rows:
+        r.normal_()
+    cache.extend([(b, ctx) for b in range(rows)])
+    lens, table = (t.to(dev) for t in cache.tables(list(range(rows))))
+    pos, slot = lens - 1, torch.tensor([int(cache.cache_rows(b, ctx - 1, 1)) for b in range(rows)], dtype=torch.int32, device=dev)
+    rope = m._rope[W.layers[0].spec.mixer.rot.key()]
+    h = torch.randn(W.layers[0].width // 8, rows, 8, device=dev).to(m.dtype)
+    x, ids = torch.randn(rows, WIDTH, device=dev), torch.arange(rows, device=dev)
+    act = torch.randn(W.layers[0].w_out.k // 8, rows, 8, device=dev).to(m.dtype)
+    raw, ss = ol.input_projection(h, W.layers[0].w_in, g.n_raw, act, g.H * g.V)
+    qn, q = ol.query_and_append(raw, ss, W.layers[0].w_uq, g, W.layers[0].q_norm, W.layers[0].kv_norm, 1e-5, rope, pos, slot, cache.rows[0])
+    o = torch.randn(rows, g.H, g.C, device=dev).to(m.dtype)
+    side = W.side_table(0)
+    sg = ol.token_gate_linear(x, W.layers[0].side_gate, side, ids, 256)
+    y = ol.linear_f32(sg, W.layers[0].side_proj, WIDTH)
+
+    def wb(w):
+        return 2 * w.packed.numel()
+    L, R, ctxs = W.layers, rows, dict(ctx=ctx)
+    k0 = L[0]
+    out = [
+        _kernel(R, "befidra", "finish (norm)", [lambda: ol.finish(x, k0.norm1, 1e-5, WIDTH, m.dtype, y=y, y_w=k0.side_norm, octets=True)] * 4,
+                R * WIDTH * 14, like="rmsnorm"),
+        _kernel(R, "befidra", "input projections", [lambda l=l: ol.input_projection(h, l.w_in, g.n_raw, act, g.H * g.V) for l in L],
+                wb(k0.w_in), 2.0 * R * k0.w_in.n * k0.w_in.k, like="gate|up"),
+        _kernel(R, "befidra", "query up + cache append",
+                [lambda l=l: ol.query_and_append(raw, ss, l.w_uq, g, l.q_norm, l.kv_norm, 1e-5, rope, pos, slot, cache.rows[0]) for l in L],
+                wb(k0.w_uq), like="o"),
+        _kernel(R, "befidra", "query to latent", [lambda l=l: ol.query_to_latent(qn, l.w_uk_t, q, g) for l in L], wb(k0.w_uk_t)),
+        _kernel(R, "befidra", "latent to value + gate", [lambda l=l: ol.latent_to_value(o, l.w_uv, raw, g.gate_off, act, g) for l in L],
+                wb(k0.w_uv)),
+        _kernel(R, "befidra", "output + down", [lambda l=l: ol.add_linear(act, l.w_out, x) for l in L], wb(k0.w_out),
+                2.0 * R * k0.w_out.n * k0.w_out.k, like="down"),
+        _kernel(R, "befidra", "token gate", [lambda l=l: ol.token_gate_linear(x, l.side_gate, side, ids, 256) for l in L], wb(k0.side_gate)),
+        _kernel(R, "befidra", "token projection", [lambda l=l: ol.linear_f32(sg, l.side_proj, WIDTH) for l in L], wb(k0.side_proj)),
+        _kernel(R, "befidra", "logits", [lambda: ol.linear_f32(h, W.logits, m.vocab_size)] * 2, wb(W.logits), like="lm_head"),
+        _kernel(R, "befidra", "attention (+ merge)",
+                [lambda c=c: ol.attn_decode(q, c, table, lens, g, k0.scale, ctx) for c in cache.rows],
+                2.0 * R * ctx * g.row, 2.0 * R * g.H * ctx * (g.row + g.C), like="attention", **ctxs),
+    ]
+    return out
+
+
+def llama_decode_kernels(m, rows, ctx):
+    from triforce_amd import ops
+    from triforce_amd.models.cache import FlashSimpleCache
+    W, dev = m.weights, m.device
+    cache = FlashSimpleCache(m, ctx + 64)
+    cache.k.normal_()
+    cache.v.normal_()
+    x = torch.randn(rows, WIDTH, device=dev).half()
+    D = WIDTH // HEADS
+    pos = torch.arange(ctx - rows, ctx, device=dev)
+    ss = ops.ss_buffer(WIDTH, dev)
+    a, act = torch.randn(rows, WIDTH, device=dev).half(), torch.randn(rows, FF, device=dev).half()
+    ops.linear(a, W.wo[0], resid=x, out=x, ss_out=ss)
+    q = torch.randn(rows, HEADS, D, device=dev).half()
+    n, R = range(LAYERS), rows
+    return [
+        _kernel(R, "llama", "rmsnorm", [lambda: ops.rmsnorm(x, W.ln1[0], 1e-5)] * 4, R * WIDTH * 4),
+        _kernel(R, "llama", "q|k|v + rope + append",
+                [lambda i=i: ops.qkv_rope(x, W.wqkv[i], W.ln1[i], 1e-5, m.cos, m.sin, pos, *cache.layer_kv(i), ctx - rows, HEADS, D, ss_in=ss)
+                 for i in n], 6.0 * WIDTH * WIDTH),
+        _kernel(R, "llama", "o", [lambda i=i: ops.linear(a, W.wo[i], resid=x, out=x, ss_out=ss) for i in n], 2.0 * WIDTH * WIDTH),
+        _kernel(R, "llama", "gate|up", [lambda i=i: ops.mlp_act(x, W.wgu[i], ln=W.ln2[i], eps=1e-5, ss_in=ss) for i in n], 4.0 * WIDTH * FF),
+        _kernel(R, "llama", "down", [lambda i=i: ops.linear(act, W.wd[i], resid=x, out=x, ss_out=ss) for i in n], 2.0 * WIDTH * FF),
+        _kernel(R, "llama", "lm_head", [lambda: ops.linear(x, W.lm_head, out_f32=True, ln=W.norm, eps=1e-5, ss_in=ss)] * 2, 2.0 * 32000 * WIDTH),
+        _kernel(R, "llama", "attention", [lambda i=i: ops.attn_decode(q, *cache.layer_kv(i), ctx, m.scale) for i in n],
+                4.0 * ctx * WIDTH, 4.0 * R * ctx * WIDTH, ctx=ctx),
+    ]
+
+
+# ---- prefill attention ------------------------------------------------------------------------------------------------------
+def prefill_kernels(bm, lm, new, past):
+    from triforce_amd import ops, ops_latent as ol
+    from triforce_amd.models.cache import FlashSimpleCache, LatentCache
+    dev, W = bm.device, bm.weights
+    L0, g = W.layers[0], W.layers[0].geom
+    nk = new + past
+    cache = LatentCache(bm, max_budget=nk, max_batch=1)
+    cache.rows[0].normal_()
+    if past:
+        cache.extend([("s", past)])
+    b = cache.plan_prefill([("s", new, [])])
+    rope = bm._rope[L0.spec.mixer.rot.key()]
+    r = lambda *s: torch.randn(*s, device=dev).to(bm.dtype)
+    q, kv, ck, y = r(new, g.H * (g.N + g.R)), r(nk, g.H * (g.N + g.V)), r(nk, g.row), r(new, L0.w_in.n)
+    act, x = r(new, L0.w_out.k), torch.randn(new, WIDTH, device=dev)
+    d, ids = r(new, WIDTH), torch.arange(new, device=dev) % 32000
+    flops = 2.0 * (new * past + new * (new + 1) / 2) * g.H * (g.N + g.R + g.V)
+    i = dict(new=new, past=past)
+    _kernel(new, "befidra", "prefill attention", [lambda: ol.attn_prefill(q, kv, ck, b.seq, new, b.pos, rope, y[:, g.gate_off:], act, g, L0.scale)] * 2,
+            2.0 * (q.numel() + kv.numel() + nk * g.R + 2 * new * g.H * g.V), flops, like="prefill attention", **i)
+    _kernel(new, "befidra", "prepare", [lambda: ol.prepare(y, g, g.n_raw, FF, L0.q_norm, L0.kv_norm, 1e-5, rope, b.pos, b.slot, cache.rows[0], act,
+                                                           g.H * g.V, want_rows=True)] * 2,
+            2.0 * new * (2 * (g.Q + FF) + 3 * g.row), like="rope + append", **i)
+    _kernel(new, "befidra", "residual", [lambda: ol.residual(d, x, True)] * 2, new * WIDTH * 12.0, **i)
+    _kernel(new, "befidra", "finish (norm)", [lambda: ol.finish(x, L0.norm1, 1e-5, WIDTH, bm.dtype, y=d, y_w=L0.side_norm)] * 2,
+            new * WIDTH * 12.0, like="rmsnorm", **i)
+    c = FlashSimpleCache(lm, nk)
+    c.k.normal_()
+    c.v.normal_()
+    lq = torch.randn(new, HEADS, WIDTH // HEADS, device=dev).half()
+    _kernel(new, "llama", "prefill attention", [lambda: ops.attn_prefill(lq, *c.layer_kv(0), nk, lm.scale)] * 2,
+            2.0 * (2 * lq.numel() + 2 * nk * WIDTH), 4.0 * (new * past + new * (new + 1) / 2) * WIDTH, **i)
+    hx = torch.randn(new, WIDTH, device=dev).half()
+    _kernel(new, "llama", "rmsnorm", [lambda: ops.rmsnorm(hx, lm.weights.ln1[0], 1e-5, residual=lq.view(new, WIDTH), sum_out=hx)] * 2, new * WIDTH * 8.0, **i)
+    qkv = torch.randn(new, 3 * WIDTH, device=dev).half()
+    pos = torch.arange(past, nk, device=dev)
+    _kernel(new, "llama", "rope + append", [lambda: ops.rope_append(qkv, lm.cos, lm.sin, pos, *c.layer_kv(0), past, HEADS, WIDTH // HEADS)] * 2,
+            new * WIDTH * 12.0, **i)
+
+
+# ---- whole models -----------------------------------------------------------------------------------------------------------
+def _seconds(fn, n):
+    torch.cuda.synchronize()
+    t0 = time.time()
+    for _ in range(n):
+        fn()
+    torch.cuda.synchronize()
+    return (time.time() - t0) / n
+
+
+def befidra_throughput(m, prompt, batch, decode_steps=64):
+    from triforce_amd.models.cache import LatentCache
+    from triforce_amd.utils.batch_infer import BatchInferenceEngine
+    from triforce_amd.utils.graph_infer import PREFILL_CHUNK
+    cache = LatentCache(m, max_budget=batch * (prompt + decode_steps + 80), max_batch=batch)
+    e = BatchInferenceEngine(m, cache)
+    toks = torch.randint(0, m.vocab_size, (batch, prompt), generator=torch.Generator().manual_seed(1)).tolist()
+
+    def fill():
+        e.clear_kv()
+        for b in range(batch):                       # (a prompt per forward: equal work per token to the single-sequence engine)
+            e.step([(b, toks[b], [prompt - 1])])
+    fill()
+    t_pre = _seconds(fill, 1)
+    ids = torch.zeros(batch, dtype=torch.int64, device=m.device)
+    names = list(range(batch))
+    for _ in range(4):
+        e.decode(names, ids)
+    t_dec = _seconds(lambda: e.decode(names, ids), decode_steps)
+    row = dict(kind="throughput", model="befidra", layers=LAYERS, prompt=prompt, batch=batch, prefill_tokens_per_s=round(batch * prompt / t_pre),
+               decode_ms_per_step=round(1e3 * t_dec, 4), decode_tokens_per_s=round(batch / t_dec, 1), prefill_chunk=PREFILL_CHUNK)
+    _emit(row)
+    return row
+
+
+def llama_throughput(m, prompt, decode_steps=64):
+    from triforce_amd.models.cache import FlashSimpleCache
+    from triforce_amd.utils import graph_infer
+    cache = FlashSimpleCache(m, prompt + decode_steps + 16)
+    ids = torch.randint(0, 32000, (1, prompt), generator=torch.Generator().manual_seed(1)).to(m.device)
+
+    def fill():
+        cache.reset()
+        graph_infer.chunked_prefill(lambda i, last_rows=None: m.forward(i, cache, last_rows=last_rows).logits, ids)
+
+    class Eng:
+        model, kv_cache = m, cache
+    with torch.inference_mode():
+        fill()
+        t_pre = _seconds(fill, 1)
+        tg = graph_infer._TargetGraph(Eng, 1, None, 2, False, 1.0, 1.0)
+        cache.seq_len = prompt
+        tok = ids[:, :1].clone()
+        for _ in range(4):
+            tg(tok)
+        t_dec = _seconds(lambda: tg(tok), decode_steps)
+    row = dict(kind="throughput", model="llama", layers=LAYERS, prompt=prompt, batch=1, prefill_tokens_per_s=round(prompt / t_pre),
+               decode_ms_per_step=round(1e3 * t_dec, 4), decode_tokens_per_s=round(1 / t_dec, 1))
+    _emit(row)
+    return row
+
+
+def run_design(args):
+    device = torch.device("cuda:0")
+    bm, lm = befidra_model(device), llama_model(device)
+    rows = []
+    for prompt in (4096, 32768):
+        rows.append(llama_throughput(lm, prompt))
+        for batch in ((1, 8, 32) if prompt == 4096 else (1, 8)):
+            rows.append(befidra_throughput(bm, prompt, batch))
+    with torch.inference_mode():
+        for r, ctx in ((1, 32768), (8, 4096), (8, 32768), (32, 4096)):
+            befidra_decode_kernels(bm, r, ctx)
+        for r, ctx in ((1, 32768), (8, 32768), (32, 4096), (1, 124928)):
+            llama_decode_kernels(lm, r, ctx)
+        for new, past in ((4096, 0), (4096, 28672)):
+            prefill_kernels(bm, lm, new, past)
+    best = max((r for r in rows if r["model"] == "befidra"), key=lambda r: r["decode_tokens_per_s"])
+    _emit(dict(metric="Befidra decode throughput, 7B-sized layers (random weights)", value=best["decode_tokens_per_s"], unit="tokens/s",
+               n_gpus=1, higher_is_better=True, dtype="bf16", data="synthetic", vs_baseline=None,
+               config=dict(model=f"befidra-7B layers x {LAYERS}", global_batch=best["batch"], seq_len=best["prompt"], parallelism="none")))
+    return 0

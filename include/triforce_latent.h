@@ -28,15 +28,18 @@ extern "C" {
 
 int tfl_abi_version(void);
 
+/* Activation blocks: element (m, k) lives at m*ld + (k/8)*oct + k%8.  Row-major rows have oct = 8; decode keeps its norm output
+ * and the output projection's input octet-major (ld = 8, oct = 8 * rows), where a 16-row operand is four contiguous runs. */
+
 /* What a skinny GEMM does with its fp32 result (row m of x, output n of the group). */
 enum {
     TFL_EPI_F32 = 0,                /* out_f[m*ld_f + n] = acc, n < n_real */
     TFL_EPI_IN = 1,                 /* n < n_raw: out_f[m*ld_f + n] = acc and ss[m*(n_raw/16) + n/16] = sum over the panel of
-                                       acc^2; else out_t[m*ld_t + n - n_raw] = gelu_tanh(acc) */
+                                       acc^2; else out_t(m, n - n_raw) = gelu_tanh(acc) */
     TFL_EPI_QUERY = 2,              /* heads of N + R outputs: out_t2[(m*H + h)*N + n] unrotated;
                                        out_t[(m*H + h)*(C + R) + C + n] rotated at pos[m] */
     TFL_EPI_LATENT = 3,             /* group h: out_t[(m*H + h)*(C + R) + n] = acc */
-    TFL_EPI_GATED = 4,              /* group h: out_t[m*ld_t + h*ppg*16 + n] = acc * sigmoid(gate[m*ld_gate + h*ppg*16 + n]) */
+    TFL_EPI_GATED = 4,              /* group h: out_t(m, h*ppg*16 + n) = acc * sigmoid(gate[m*ld_gate + h*ppg*16 + n]) */
     TFL_EPI_RESIDUAL = 5,           /* out_f[m*ld_f + n] += acc */
     TFL_EPI_TOKEN = 6               /* out_t[m*ld_t + n] = gelu_tanh(acc) * tok_table[ids[m]*ld_tok + n], n < n_real (0 behind) */
 };
@@ -63,7 +66,7 @@ typedef struct TflGemm {
     const float* kv_norm_w;         /* fp32 [C] */
     void* cache;                    /* [cache rows][C + R] */
     const int32_t* slot;            /* cache row per batch row; negative: nothing is stored */
-    int64_t ld_x, x_group, ld_t, ld_f, ld_gate, ld_tok, ld_kv;
+    int64_t ld_x, x_oct, x_group, ld_t, t_oct, ld_f, ld_gate, ld_tok, ld_kv;
     int32_t rows, n, k, groups;     /* n = outputs per group, all groups alike */
     int32_t n_real, k_real, n_raw, ss_n, ss_ld;
     int32_t H, N, R, C, half, c_real, max_pos, cache_rows, vocab;
@@ -77,10 +80,10 @@ int tfl_gemm(const TflGemm* a, int dtype, int x_mode, int epilogue, void* stream
  *   x += y / rms(y) * y_w     (y != NULL; fp32 when y_f32, else T)
  *   x += step                 (step != NULL)
  *   h = x / rms(x) * norm_w   (T)
- * width_real elements carry data, rows have stride width (padded with zeros). */
+ * width_real elements carry data, rows have stride width (padded with zeros); h is an activation block (below). */
 int tfl_finish(const void* embed, const int64_t* ids, int vocab, const void* y, int y_f32, int64_t ld_y, const float* y_w,
-               const float* step, const float* norm_w, float* x, void* h, int rows, int width, int width_real, float eps,
-               int dtype, void* stream);
+               const float* step, const float* norm_w, float* x, void* h, int64_t ld_h, int64_t h_oct, int rows, int width,
+               int width_real, float eps, int dtype, void* stream);
 
 /* x += d (T); xt = T(x)  (xt may be NULL). */
 int tfl_residual(const void* d, float* x, void* xt, int64_t n, int dtype, void* stream);

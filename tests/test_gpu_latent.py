@@ -55,20 +55,27 @@ def f(t):
 ROWS = [1, 3, 16, 17, 33, 70]
 
 
+def octets(x):
+    rows, k = x.shape
+    return x.view(rows, k // 8, 8).permute(1, 0, 2).contiguous()
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("rows", ROWS)
-@pytest.mark.parametrize("n,k,n_real", [(32, 32, 17), (96, 416, 96), (2080, 96, 2077)])
+@pytest.mark.parametrize("n,k,n_real", [(32, 32, 17), (96, 416, 96), (2080, 96, 2077), (5024, 1056, 5001), (10272, 64, 10272), (13472, 160, 13469)])
 def test_linear_f32(ol, dtype, rows, n, k, n_real):
     w, x = rnd(n, k, seed=1, dtype=dtype), rnd(rows, k, seed=2, dtype=dtype)
-    y = ol.linear_f32(x, ol.TileWeight(w), n_real)
+    wt = ol.TileWeight(w)
+    y = ol.linear_f32(x, wt, n_real)
+    assert torch.equal(ol.act_rows(octets(x)), x) and torch.equal(ol.linear_f32(octets(x), wt, n_real), y)
     torch.testing.assert_close(y, (f(x) @ f(w).T)[:, :n_real], atol=2e-4 * k ** 0.5, rtol=1e-4)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("rows", ROWS)
-@pytest.mark.parametrize("n_up", [0, 96])
-def test_input_projection(ol, dtype, rows, n_up):
-    k, n_raw, off = 160, 224, 64
+@pytest.mark.parametrize("n_raw,n_up", [(224, 0), (224, 96), (224, 13312)])
+def test_input_projection(ol, dtype, rows, n_raw, n_up):
+    k, off = 160, 64
     w, x = rnd(n_raw + n_up, k, seed=1, dtype=dtype, scale=k ** -0.5), rnd(rows, k, seed=2, dtype=dtype)
     act = torch.full((rows, off + n_up), 7.0, dtype=dtype, device=DEV)
     raw, ss = ol.input_projection(x, ol.TileWeight(w), n_raw, act, off)
@@ -77,6 +84,9 @@ def test_input_projection(ol, dtype, rows, n_up):
     torch.testing.assert_close(ss, want[:, :n_raw].view(rows, -1, 16).pow(2).sum(-1), atol=1e-3, rtol=1e-3)
     torch.testing.assert_close(f(act[:, off:]), R.gelu(want[:, n_raw:]), **OP[dtype])
     assert bool((act[:, :off] == 7).all())
+    block = torch.full(((off + n_up) // 8, rows, 8), 7.0, dtype=dtype, device=DEV)
+    raw2, ss2 = ol.input_projection(octets(x), ol.TileWeight(w), n_raw, block, off)
+    assert torch.equal(ol.act_rows(block), act) and torch.equal(raw2, raw) and torch.equal(ss2, ss)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -128,14 +138,19 @@ def test_per_head_projections_and_gate(ol, dtype, rows):
     want = torch.stack([f(o[:, h]) @ f(uv[h]).T for h in range(g.H)], 1).reshape(rows, -1) * torch.sigmoid(raw[:, 64:])
     torch.testing.assert_close(f(act[:, :g.H * g.V]), want, **OP[dtype])
     assert bool((act[:, g.H * g.V:] == 3).all())
+    block = torch.full((act.shape[1] // 8, rows, 8), 3.0, dtype=dtype, device=DEV)
+    ol.latent_to_value(o, ol.TileWeight(uv), raw, 64, block, g)
+    assert torch.equal(ol.act_rows(block), act)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("rows", ROWS)
 def test_residual_and_token_gemms(ol, dtype, rows):
     w, a, x = rnd(96, 160, seed=1, dtype=dtype), rnd(rows, 160, seed=2, dtype=dtype), rnd(rows, 96, seed=3)
-    want = x + f(a) @ f(w).T
+    want, x2 = x + f(a) @ f(w).T, x.clone()
     ol.add_linear(a, ol.TileWeight(w), x)
+    ol.add_linear(octets(a), ol.TileWeight(w), x2)
+    assert torch.equal(x, x2)
     torch.testing.assert_close(x, want, atol=1e-3, rtol=1e-4)
     w, table = rnd(32, 96, seed=4, dtype=dtype, scale=0.1), rnd(50, 60, seed=5, dtype=dtype)
     ids = torch.randint(0, 50, (rows,), generator=torch.Generator().manual_seed(1)).to(DEV)
@@ -166,6 +181,8 @@ def test_finish(ol, dtype, real, width, parts):
         h = ol.finish(got, nw, eps, real, dtype, embed=emb if "embed" in parts else None, ids=ids if "embed" in parts else None,
                       y=y if "y" in parts else None, y_w=yw if "y" in parts else None, step=step if "step" in parts else None)
         torch.testing.assert_close(got, want, atol=1e-5, rtol=1e-5)
+        h2 = ol.finish(got.clone(), nw, eps, real, dtype, octets=True)
+        torch.testing.assert_close(f(ol.act_rows(h2)), f(h), atol=1e-6, rtol=1e-2)
         torch.testing.assert_close(f(h), want / torch.sqrt(want.pow(2).sum(-1, keepdim=True) / real + eps) * nw, **OP[dtype])
 
 

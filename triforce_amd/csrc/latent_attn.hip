@@ -19,8 +19,8 @@
 // Weights as two bfloat16 (value and remainder): the PV product then sees them to 16 bits like the fp32 softmax made them.
 template <typename T> struct DecodeCfg { static constexpr int PARTS = sizeof(T) == 2 ? 2 : 1; };
 
-// WC > 0: chunks (W / 32) at compile time with the register look-ahead; 0: any width up to the LDS limit.
-template <typename T, int NW, int HT, int NTW, int WC>
+// Any sizes up to the LDS limit.
+template <typename T, int NW, int HT, int NTW>
 __global__ __launch_bounds__(NW * 64, 1) void attn_latent_kernel(const T* __restrict__ q, const T* __restrict__ cache, int n_pages,
                                                               const int32_t* __restrict__ table, int table_ld,
                                                               const int32_t* __restrict__ len, T* __restrict__ out,
@@ -30,8 +30,7 @@ __global__ __launch_bounds__(NW * 64, 1) void attn_latent_kernel(const T* __rest
     constexpr int KT = 16 * NW, NT = NW * 64, EPV = 16 / sizeof(T), PADE = EPV;
     constexpr int PARTS = DecodeCfg<T>::PARTS;
     extern __shared__ __align__(16) char smem[];
-    [[maybe_unused]] const int wc = (C + R) >> 5;
-    const int W = C + R, ldk = (WC ? WC * 32 : W) + PADE, ldp = KT + PADE;
+    const int W = C + R, wc = W >> 5, ldk = W + PADE, ldp = KT + PADE;
     T* Kt = (T*)smem;                                         // [KT][ldk]
     T* Qs = Kt + KT * ldk;                                    // [16 HT][ldk]
     T* Ps = Qs + 16 * HT * ldk;                               // [PARTS][16 HT][ldp]
@@ -42,7 +41,7 @@ __global__ __launch_bounds__(NW * 64, 1) void attn_latent_kernel(const T* __rest
     const int ntiles = n > 0 ? (n + KT - 1) / KT : 0;
     const int per = (ntiles + nsplit - 1) / nsplit;
     const int t_beg = min(split * per, ntiles), t_end = min(ntiles, t_beg + per);
-    const int ppr = (WC ? WC * 32 : W) / EPV;                 // 16-byte pieces per row
+    const int ppr = W / EPV;                 // 16-byte pieces per row
     const int32_t* tab = table + (int64_t)row * table_ld;
 
     for (int p = tid; p < 16 * HT * ppr; p += NT) {           // queries of this head group (heads past H: zeros)
@@ -51,19 +50,11 @@ __global__ __launch_bounds__(NW * 64, 1) void attn_latent_kernel(const T* __rest
         if (h0 + r < H) v = *reinterpret_cast<const uint4*>(q + ((int64_t)row * H + h0 + r) * W + EPV * c);
         *reinterpret_cast<uint4*>(Qs + r * ldk + EPV * c) = v;
     }
-    constexpr int NPRE = WC ? (KT * WC * 32 / EPV) / NT : 1;  // pieces per thread and tile
-    uint4 pre[NPRE];
     auto page_base = [&](int t) {
         const int k0 = t * KT;
         int pg = tab[k0 / TFL_PAGE];
         pg = pg < 0 ? 0 : (pg >= n_pages ? n_pages - 1 : pg);
         return (int64_t)pg * TFL_PAGE + (k0 & (TFL_PAGE - 1));
-    };
-    auto fetch = [&](int t) {
-        const T* base = cache + page_base(t) * W;
-#pragma unroll
-        for (int j = 0; j < NPRE; ++j)
-            pre[j] = *reinterpret_cast<const uint4*>(base + (int64_t)(tid + j * NT) * EPV);
     };
     f32x4 o[HT][NTW];
     float m_run[HT], l_run[HT];
@@ -74,28 +65,16 @@ __global__ __launch_bounds__(NW * 64, 1) void attn_latent_kernel(const T* __rest
 #pragma unroll
         for (int t = 0; t < NTW; ++t) o[h][t] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
-    if (WC && t_beg < t_end) fetch(t_beg);
     for (int t = t_beg; t < t_end; ++t) {
         const int k0 = t * KT;
-        if constexpr (WC > 0) {
-#pragma unroll
-            for (int j = 0; j < NPRE; ++j) {
-                const int p = tid + j * NT, r = p / ppr, c = p - r * ppr;
-                uint4 v = pre[j];
-                if (k0 + r >= n) v = uint4{0, 0, 0, 0};       // rows past the end: never let stale contents into 0 * x
-                *reinterpret_cast<uint4*>(Kt + r * ldk + EPV * c) = v;
-            }
-        } else {
-            const T* base = cache + page_base(t) * W;
-            for (int p = tid; p < KT * ppr; p += NT) {
-                const int r = p / ppr, c = p - r * ppr;
-                uint4 v = {0, 0, 0, 0};
-                if (k0 + r < n) v = *reinterpret_cast<const uint4*>(base + (int64_t)r * W + EPV * c);
-                *reinterpret_cast<uint4*>(Kt + r * ldk + EPV * c) = v;
-            }
+        const T* base = cache + page_base(t) * W;
+        for (int p = tid; p < KT * ppr; p += NT) {
+            const int r = p / ppr, c = p - r * ppr;
+            uint4 v = {0, 0, 0, 0};
+            if (k0 + r < n) v = *reinterpret_cast<const uint4*>(base + (int64_t)r * W + EPV * c);
+            *reinterpret_cast<uint4*>(Kt + r * ldk + EPV * c) = v;
         }
         __syncthreads();
-        if (WC && t + 1 < t_end) fetch(t + 1);
         f32x4 s[HT];
 #pragma unroll
         for (int h = 0; h < HT; ++h) s[h] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -106,12 +85,7 @@ __global__ __launch_bounds__(NW * 64, 1) void attn_latent_kernel(const T* __rest
 #pragma unroll
             for (int h = 0; h < HT; ++h) s[h] = El<T>::mma(a, load_frag(qp + h * 16 * ldk + 32 * c), s[h]);
         };
-        if constexpr (WC > 0) {
-#pragma unroll 6
-            for (int c = 0; c < WC; ++c) chunk(c);
-        } else {
-            for (int c = 0; c < wc; ++c) chunk(c);
-        }
+        for (int c = 0; c < wc; ++c) chunk(c);
 #pragma unroll
         for (int h = 0; h < HT; ++h) {
             float mx = NEG_INF;
@@ -219,17 +193,17 @@ __global__ __launch_bounds__(NW * 64, 1) void attn_latent_kernel(const T* __rest
     }
 }
 
-// Merge of the splits: one workgroup per (head, row).
+// Merge of the splits: one workgroup per (64 latent columns, head, row); 16 threads across the columns, 16 over the splits.
 template <typename T>
 __global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restrict__ ws, T* __restrict__ out, int rows, int H,
                                                            int C, int nsplit) {
     __shared__ float wgt[256];
+    __shared__ float red[8];
     __shared__ f32x4 acc[256];
-    const int head = blockIdx.x, row = blockIdx.y, tid = threadIdx.x;
+    const int head = blockIdx.y, row = blockIdx.z, tid = threadIdx.x;
     const int64_t at = ((int64_t)row * H + head) * nsplit;
     const float* ml = ws + (int64_t)rows * H * nsplit * C + at * 2;
-    // thread s owns split s (nsplit <= 256); an empty split has weight 0 and its partial row is never read
-    __shared__ float red[8];
+    // thread s owns the statistics of split s (nsplit <= 256); an empty split has weight 0 and its partial row is never read
     const float ls = tid < nsplit ? ml[2 * tid + 1] : 0.f;
     const float ms = ls > 0.f ? ml[2 * tid] : NEG_INF;
     float m = ms;
@@ -239,32 +213,216 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restri
     __syncthreads();
     m = fmaxf(fmaxf(red[4], red[5]), fmaxf(red[6], red[7]));
     const float w = ls > 0.f ? exp2f((ms - m) * LOG2E) : 0.f;
-    const float l = block_sum256(w * ls, red);
+    const float l = block_sum<4>(w * ls, red);
     wgt[tid] = l > 0.f ? w / l : 0.f;
     __syncthreads();
-    const int nq = C >> 2, lanes = nq < 256 ? nq : 256, grps = 256 / lanes;      // groups of threads share the splits
-    const int gi = tid / lanes, li = tid - gi * lanes;
-    for (int q0 = 0; q0 < nq; q0 += lanes) {
-        const int q = q0 + li;
-        f32x4 v = {0.f, 0.f, 0.f, 0.f};
-        if (gi < grps && q < nq)
-            for (int s = gi; s < nsplit; s += grps)
-                if (wgt[s] > 0.f) {
-                    const f32x4 z = *reinterpret_cast<const f32x4*>(ws + (at + s) * C + 4 * q);
+    const int col = 64 * blockIdx.x + 4 * (tid & 15), grp = tid >> 4;
+    f32x4 v = {0.f, 0.f, 0.f, 0.f};
+    if (col < C) {
+        const float* src = ws + at * C + col;
+#pragma unroll 4
+        for (int s = grp; s < nsplit; s += 16) {
+            const float ws_ = wgt[s];
+            if (ws_ > 0.f) {
+                const f32x4 z = *reinterpret_cast<const f32x4*>(src + (int64_t)s * C);
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) v[r] = fmaf(z[r], wgt[s], v[r]);
-                }
-        acc[tid] = v;
-        __syncthreads();
-        if (gi == 0 && q < nq) {
-            for (int k = 1; k < grps; ++k) {
-                const f32x4 z = acc[k * lanes + li];
-#pragma unroll
-                for (int r = 0; r < 4; ++r) v[r] += z[r];
+                for (int r = 0; r < 4; ++r) v[r] = fmaf(z[r], ws_, v[r]);
             }
-            store_quad(out + ((int64_t)row * H + head) * C + 4 * q, v);
         }
+    }
+    acc[tid] = v;
+    __syncthreads();
+    if (grp == 0 && col < C) {
+#pragma unroll
+        for (int k = 1; k < 16; ++k) {
+            const f32x4 z = acc[16 * k + tid];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v[r] += z[r];
+        }
+        store_quad(out + ((int64_t)row * H + head) * C + col, v);
+    }
+}
+
+// The same attention for a known row size (WC chunks of 32, the first CT 16-wide tiles of it latent), bfloat16, HT head tiles of
+// 16 per workgroup and four waves per head tile: wave (ht, ks) scores keys 16 ks .. of its head tile with the queries held in
+// registers, and accumulates CT / (4 HT) of the latent tiles for all heads.  Two pages in LDS: the next one is written and the one
+// after it requested while the current one is used, so a page costs two barriers and the stream never waits for the arithmetic.
+template <int HT, int WC, int CT>
+__global__ __launch_bounds__(256 * HT, HT) void attn_latent_sized_kernel(const bf16* __restrict__ q, const bf16* __restrict__ cache,
+                                                                         int n_pages, const int32_t* __restrict__ table, int table_ld,
+                                                                         const int32_t* __restrict__ len, bf16* __restrict__ out,
+                                                                         float* __restrict__ ws, int H, float scale, int nsplit,
+                                                                         int rows) {
+    constexpr int NT = 256 * HT, W = 32 * WC, C = 16 * CT, LDK = W + 8, LDP = 64 + 8, NTW = CT / (4 * HT), NPRE = 64 * (W / 8) / NT;
+    static_assert(CT % (4 * HT) == 0 && 64 * (W / 8) % NT == 0, "tile split");
+    extern __shared__ __align__(16) char smem[];
+    bf16* Kt = (bf16*)smem;                                   // [2][64][LDK]
+    bf16* Ps = Kt + 2 * 64 * LDK;                             // [2 (value, remainder)][16 HT][LDP]
+    float* red = (float*)(Ps + 2 * 16 * HT * LDP);            // [4][16 HT]
+    const int split = blockIdx.x, h0 = blockIdx.y * 16 * HT, row = blockIdx.z;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g = lane >> 4, i = lane & 15, ks = wave & 3, ht = wave >> 2;
+    const int n = len[row];
+    const int ntiles = n > 0 ? (n + 63) / 64 : 0;
+    const int per = (ntiles + nsplit - 1) / nsplit;
+    const int t_beg = min(split * per, ntiles), t_end = min(ntiles, t_beg + per);
+    const int32_t* tab = table + (int64_t)row * table_ld;
+
+    bf16x8 qf[WC];
+    {
+        const int head = h0 + 16 * ht + i;
+        const bf16* src = q + ((int64_t)row * H + min(head, H - 1)) * W + 8 * g;
+#pragma unroll
+        for (int c = 0; c < WC; ++c) {
+            qf[c] = load_frag(src + 32 * c);
+            if (head >= H) qf[c] = bf16x8{};
+        }
+    }
+    uint4 pre[NPRE];
+    auto page_of = [&](int t) {
+        const int pg = tab[t];
+        return pg < 0 ? 0 : (pg >= n_pages ? n_pages - 1 : pg);
+    };
+    auto fetch = [&](int pg) {
+        const bf16* base = cache + (int64_t)pg * (64 * W) + tid * 8;
+#pragma unroll
+        for (int j = 0; j < NPRE; ++j) pre[j] = *reinterpret_cast<const uint4*>(base + j * NT * 8);
+    };
+    auto put = [&](int t) {
+        bf16* dst = Kt + (t & 1) * 64 * LDK;
+        const bool edge = 64 * t + 64 > n;
+#pragma unroll
+        for (int j = 0; j < NPRE; ++j) {
+            const int p = tid + j * NT, r = p / (W / 8), c = p - r * (W / 8);
+            uint4 v = pre[j];
+            if (edge && 64 * t + r >= n) v = uint4{0, 0, 0, 0};     // rows past the end: never let stale contents into 0 * x
+            *reinterpret_cast<uint4*>(dst + r * LDK + 8 * c) = v;
+        }
+    };
+    f32x4 o[HT][NTW];
+    float m_run[HT], l_run = 0.f;
+#pragma unroll
+    for (int h = 0; h < HT; ++h) {
+        m_run[h] = NEG_INF;
+#pragma unroll
+        for (int x = 0; x < NTW; ++x) o[h][x] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    int pg_next = 0;
+    if (t_beg < t_end) {
+        fetch(page_of(t_beg));
+        if (t_beg + 1 < t_end) pg_next = page_of(t_beg + 1);
+        put(t_beg);
+        if (t_beg + 1 < t_end) fetch(pg_next);
+        if (t_beg + 2 < t_end) pg_next = page_of(t_beg + 2);
         __syncthreads();
+    }
+    for (int t = t_beg; t < t_end; ++t) {
+        const bf16* K = Kt + (t & 1) * 64 * LDK;
+        const int k0 = 64 * t;
+        f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;
+        const bf16* kp = K + (16 * ks + i) * LDK + 8 * g;
+#pragma unroll
+        for (int c = 0; c < WC; c += 2) {
+            s0 = El<bf16>::mma(load_frag(kp + 32 * c), qf[c], s0);
+            if (c + 1 < WC) s1 = El<bf16>::mma(load_frag(kp + 32 * (c + 1)), qf[c + 1], s1);
+        }
+        float mx = NEG_INF;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            s0[r] = k0 + 16 * ks + 4 * g + r < n ? (s0[r] + s1[r]) * scale : NEG_INF;
+            mx = fmaxf(mx, s0[r]);
+        }
+        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        if (g == 0) red[ks * 16 * HT + 16 * ht + i] = mx;
+        __syncthreads();                                      // maxima are in; everyone is done with the previous page and weights
+        float alpha[HT];
+#pragma unroll
+        for (int h = 0; h < HT; ++h) {
+            float m = m_run[h];
+#pragma unroll
+            for (int w = 0; w < 4; ++w) m = fmaxf(m, red[w * 16 * HT + 16 * h + i]);
+            alpha[h] = __builtin_amdgcn_exp2f((m_run[h] - m) * LOG2E);   // (the page's first key is visible: m is finite)
+            m_run[h] = m;
+        }
+        {
+            float m = m_run[0], al = alpha[0];
+#pragma unroll
+            for (int h = 1; h < HT; ++h)
+                if (ht == h) { m = m_run[h]; al = alpha[h]; }
+            f32x4 p, lo;
+            float sum = 0.f;
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                p[r] = __builtin_amdgcn_exp2f((s0[r] - m) * LOG2E);
+                sum += p[r];
+                lo[r] = p[r] - (float)(bf16)p[r];
+            }
+            l_run = l_run * al + sum;
+            bf16* dst = Ps + (16 * ht + i) * LDP + 16 * ks + 4 * g;
+            store_quad(dst, p);
+            store_quad(dst + 16 * HT * LDP, lo);
+        }
+        if (t + 1 < t_end) {
+            put(t + 1);
+            if (t + 2 < t_end) fetch(pg_next);
+            if (t + 3 < t_end) pg_next = page_of(t + 3);
+        }
+        __syncthreads();                                      // weights and the next page are in
+#pragma unroll
+        for (int h = 0; h < HT; ++h)
+#pragma unroll
+            for (int x = 0; x < NTW; ++x)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) o[h][x][r] *= alpha[h];
+#pragma unroll
+        for (int c = 0; c < 2; ++c) {
+            bf16x8 b[HT][2];
+#pragma unroll
+            for (int h = 0; h < HT; ++h)
+#pragma unroll
+                for (int z = 0; z < 2; ++z) b[h][z] = load_frag(Ps + (z * 16 * HT + 16 * h + i) * LDP + 32 * c + 8 * g);
+#pragma unroll
+            for (int x = 0; x < NTW; ++x) {
+                const bf16x8 a = load_frag_t(K, LDK, 32 * c + 8 * g, 32 * c + 8 * g + 4, 16 * (wave * NTW + x), i);
+#pragma unroll
+                for (int z = 0; z < 2; ++z)
+#pragma unroll
+                    for (int h = 0; h < HT; ++h) o[h][x] = El<bf16>::mma(a, b[h][z], o[h][x]);
+            }
+        }
+    }
+    __syncthreads();
+    l_run += __shfl_xor(l_run, 16, 64);
+    l_run += __shfl_xor(l_run, 32, 64);
+    if (g == 0) red[ks * 16 * HT + 16 * ht + i] = l_run;
+    __syncthreads();
+#pragma unroll
+    for (int h = 0; h < HT; ++h) {
+        const int head = h0 + 16 * h + i;
+        if (head >= H) continue;
+        const float l = red[16 * h + i] + red[16 * HT + 16 * h + i] + red[32 * HT + 16 * h + i] + red[48 * HT + 16 * h + i];
+        if (nsplit == 1) {
+            const float inv = l > 0.f ? 1.0f / l : 0.f;
+#pragma unroll
+            for (int x = 0; x < NTW; ++x) {
+                f32x4 v = o[h][x];
+#pragma unroll
+                for (int r = 0; r < 4; ++r) v[r] *= inv;
+                store_quad(out + ((int64_t)row * H + head) * C + 16 * (wave * NTW + x) + 4 * g, v);
+            }
+        } else {
+            const int64_t at = ((int64_t)row * H + head) * nsplit + split;
+            if (l > 0.f) {                                    // (the partial row of an empty split is not read either)
+#pragma unroll
+                for (int x = 0; x < NTW; ++x)
+                    *reinterpret_cast<f32x4*>(ws + at * C + 16 * (wave * NTW + x) + 4 * g) = o[h][x];
+            }
+            if (wave == 0 && g == 0) {
+                float* ml = ws + (int64_t)rows * H * nsplit * C + at * 2;
+                ml[0] = m_run[h];
+                ml[1] = l;
+            }
+        }
     }
 }
 
@@ -286,14 +444,14 @@ extern "C" int tfl_attn_decode_pick_nsplit(int rows, int H, int max_len) {
     return n < 1 ? 1 : n;
 }
 
-template <typename T, int NW, int HT, int NTW, int WC>
+template <typename T, int NW, int HT, int NTW>
 static int launch_latent(const void* q, const void* cache, int n_pages, const int32_t* table, int table_ld, const int32_t* len,
                          void* out, float* ws, int rows, int H, int C, int R, float scale, int nsplit, hipStream_t st) {
     const int W = C + R, pad = 16 / (int)sizeof(T), KT = 16 * NW;
     const size_t lds = sizeof(T) * ((size_t)(KT + 16 * HT) * (W + pad) + (size_t)DecodeCfg<T>::PARTS * 16 * HT * (KT + pad))
                      + sizeof(float) * NW * 16 * HT;
     if (lds > 160 * 1024) return TF_ERANGE;
-    auto k = attn_latent_kernel<T, NW, HT, NTW, WC>;
+    auto k = attn_latent_kernel<T, NW, HT, NTW>;
     static bool attr = false;
     if (!attr) {
         const hipError_t e = hipFuncSetAttribute((const void*)k, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
@@ -304,7 +462,30 @@ static int launch_latent(const void* q, const void* cache, int n_pages, const in
                        n_pages, table, table_ld, len, (T*)out, ws, H, C, R, scale, nsplit, rows);
     TFL_LAUNCH_CHECK();
     if (nsplit > 1) {
-        hipLaunchKernelGGL((latent_merge_kernel<T>), dim3(H, rows), dim3(256), 0, st, ws, (T*)out, rows, H, C, nsplit);
+        hipLaunchKernelGGL((latent_merge_kernel<T>), dim3((C + 63) / 64, H, rows), dim3(256), 0, st, ws, (T*)out, rows, H, C, nsplit);
+        TFL_LAUNCH_CHECK();
+    }
+    return TF_OK;
+}
+
+template <int HT, int WC, int CT>
+static int launch_latent_sized(const void* q, const void* cache, int n_pages, const int32_t* table, int table_ld, const int32_t* len,
+                               void* out, float* ws, int rows, int H, float scale, int nsplit, hipStream_t st) {
+    constexpr size_t lds = 2 * 64 * (32 * WC + 8) * sizeof(bf16) + 2 * 16 * HT * (64 + 8) * sizeof(bf16) + 4 * 16 * HT * sizeof(float);
+    static_assert(lds <= 160 * 1024, "LDS");
+    auto k = attn_latent_sized_kernel<HT, WC, CT>;
+    static bool attr = false;
+    if (!attr) {
+        const hipError_t e = hipFuncSetAttribute((const void*)k, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return (int)e;
+        attr = true;
+    }
+    hipLaunchKernelGGL(k, dim3(nsplit, (H + 16 * HT - 1) / (16 * HT), rows), dim3(256 * HT), lds, st, (const bf16*)q, (const bf16*)cache,
+                       n_pages, table, table_ld, len, (bf16*)out, ws, H, scale, nsplit, rows);
+    TFL_LAUNCH_CHECK();
+    if (nsplit > 1) {
+        hipLaunchKernelGGL((latent_merge_kernel<bf16>), dim3((16 * CT + 63) / 64, H, rows), dim3(256), 0, st, ws, (bf16*)out, rows, H,
+                           16 * CT, nsplit);
         TFL_LAUNCH_CHECK();
     }
     return TF_OK;
@@ -317,18 +498,21 @@ extern "C" int tfl_attn_decode(const void* q, const void* cache, int n_pages, co
     if (C < 32 || (C & 31) || R < 0 || (R & 31) || nsplit < 1 || nsplit > TFL_MAX_SPLIT) return TF_EINVAL;
     if (nsplit > 1 && (!ws || ws_floats < tfl_attn_decode_ws_floats(rows, H, C, nsplit))) return TF_ENOSPC;
     hipStream_t st = (hipStream_t)stream;
-#define GO(T, NW, HT, NTW, WC) \
-    return launch_latent<T, NW, HT, NTW, WC>(q, cache, n_pages, table, table_ld, len, out, ws, rows, H, C, R, scale, nsplit, st)
+#define GO(T, NW, HT, NTW) \
+    return launch_latent<T, NW, HT, NTW>(q, cache, n_pages, table, table_ld, len, out, ws, rows, H, C, R, scale, nsplit, st)
     if (dtype == 0) {
-        if (C == 512 && R == 64) { if (H <= 16) GO(bf16, 4, 1, 8, 18); GO(bf16, 4, 2, 8, 18); }
-        if (C <= 128) { if (H <= 16) GO(bf16, 4, 1, 2, 0); GO(bf16, 4, 2, 2, 0); }
-        if (C <= 512) { if (H <= 16) GO(bf16, 4, 1, 8, 0); GO(bf16, 4, 2, 8, 0); }
-        if (C <= 1024) GO(bf16, 2, 1, 32, 0);
+        if (C == 512 && R == 64) {
+            if (H <= 16) return launch_latent_sized<1, 18, 32>(q, cache, n_pages, table, table_ld, len, out, ws, rows, H, scale, nsplit, st);
+            return launch_latent_sized<2, 18, 32>(q, cache, n_pages, table, table_ld, len, out, ws, rows, H, scale, nsplit, st);
+        }
+        if (C <= 128) { if (H <= 16) GO(bf16, 4, 1, 2); GO(bf16, 4, 2, 2); }
+        if (C <= 512) { if (H <= 16) GO(bf16, 4, 1, 8); GO(bf16, 4, 2, 8); }
+        if (C <= 1024) GO(bf16, 2, 1, 32);
         return TF_ERANGE;
     }
     if (dtype == 1) {
-        if (C <= 128) { if (H <= 16) GO(float, 4, 1, 2, 0); GO(float, 4, 2, 2, 0); }
-        if (C <= 512) GO(float, 2, 1, 16, 0);
+        if (C <= 128) { if (H <= 16) GO(float, 4, 1, 2); GO(float, 4, 2, 2); }
+        if (C <= 512) GO(float, 2, 1, 16);
         return TF_ERANGE;
     }
 #undef GO
@@ -336,10 +520,12 @@ extern "C" int tfl_attn_decode(const void* q, const void* cache, int n_pages, co
 }
 
 // --------------------------------------------------------------------------------------------------------------- prefill
+template <int V> struct Int { static constexpr int value = V; };
+
 // KT keys per tile, QT 16-row query tiles per wave, up to DK 32-wide chunks of query-key size (NC unrotated ones first) and DV
 // 16-wide tiles of value size.  EXACT: the sizes are exactly NCX, DK, DV (no bounds in the inner loops, register look-ahead).
 template <typename T, int KT, int QT, int DK, int DV, int NCX>
-__global__ __launch_bounds__(256, 1) void attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ kv, const T* __restrict__ ck,
+__global__ __launch_bounds__(256, NCX > 0 ? 2 : 1) void attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ kv, const T* __restrict__ ck,
                                                            const int32_t* __restrict__ seq, const int32_t* __restrict__ pos,
                                                            const float* __restrict__ cosb, const float* __restrict__ sinb,
                                                            int half, int max_pos, const T* __restrict__ gate, int64_t ld_gate,
@@ -354,10 +540,13 @@ __global__ __launch_bounds__(256, 1) void attn_prefill_kernel(const T* __restric
     T* Ks = (T*)smem;                                         // [KT][ldk]
     T* Vs = Ks + KT * ldk;                                    // [KT][ldv]
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g = lane >> 4, i = lane & 15;
-    const int h = blockIdx.y;
-    const int32_t* sq = seq + 4 * blockIdx.z;
+    // workgroups go round-robin over the 8 XCDs: all query blocks of a head sit on one of them and share its L2, longest first
+    const int nqb = gridDim.x / H, id = blockIdx.x;
+    const bool by_xcd = (H & 7) == 0;
+    const int j_ = by_xcd ? id >> 3 : id, h = by_xcd ? (j_ / nqb) * 8 + (id & 7) : j_ / nqb;
+    const int32_t* sq = seq + 4 * blockIdx.y;
     const int q_at = sq[0], nq = sq[1], k_at = sq[2], nk = sq[3];
-    const int qb = (gridDim.x - 1 - blockIdx.x) * QB;         // longest blocks first
+    const int qb = (nqb - 1 - j_ % nqb) * QB;
     if (qb >= nq || nq < 1 || nk < nq || q_at < 0 || k_at < 0 || q_at + nq > tq || k_at + nk > tk) return;
     const int past = nk - nq;
     const int64_t ld_kv = (int64_t)H * (N + V), ld_ck = C + R;
@@ -402,57 +591,64 @@ __global__ __launch_bounds__(256, 1) void attn_prefill_kernel(const T* __restric
     const int last_q = min(qb + QB, nq) - 1;                  // last query row of the workgroup
     const int ntiles = (past + last_q) / KT + 1;
     const int first_qpos = past + qb + 16 * wave * QT;        // the wave's first row: tiles that end before it need no mask
-    const int kn = N / EPV, kr = R / EPV, vn = V / EPV, ppr = kn + kr + vn;   // 16-byte pieces per key
-    constexpr int NPRE = EXACT ? (KT * (32 * DK + 16 * DV) / EPV) / 256 : 1;
-    uint4 pre[NPRE];
-    auto piece = [&](int p, int t, bool zero, int& key, int& dst_v, int& dst_c) {
-        key = p / ppr;
-        int c = p - key * ppr;
-        const int64_t kk = k_at + min(t * KT + key, nk - 1);
-        const T* src;
-        if (c < kn) { src = kv + kk * ld_kv + (int64_t)h * N + EPV * c; dst_v = 0; dst_c = EPV * c; }
-        else if (c < kn + kr) { c -= kn; src = ck + kk * ld_ck + C + EPV * c; dst_v = 0; dst_c = N + EPV * c; }
-        else { c -= kn + kr; src = kv + kk * ld_kv + (int64_t)H * N + (int64_t)h * V + EPV * c; dst_v = 1; dst_c = EPV * c; }
-        uint4 v = {0, 0, 0, 0};
-        if (!zero) v = *reinterpret_cast<const uint4*>(src);
-        return v;
-    };
-    auto put = [&](int key, int dst_v, int dst_c, uint4 v) {
-        *reinterpret_cast<uint4*>(dst_v ? Vs + key * ldv + dst_c : Ks + key * ldk + dst_c) = v;
-    };
-    if constexpr (EXACT) {
+    [[maybe_unused]] const int kn = N / EPV, kr = R / EPV, vn = V / EPV, ppr = kn + kr + vn;   // 16-byte pieces per key
+    // EXACT: a tile is NJ pieces per thread; piece j of a section is row (tid / pieces per row) + j * step of it
+    constexpr int RCX = EXACT ? DK - NCX : 1, NKX = EXACT ? NCX : 1, JV = EXACT ? DV / 2 : 1, NJ = EXACT ? NKX + RCX + JV : 1;
+    static_assert(!EXACT || (KT == 64 && 256 % (4 * NKX) == 0 && 256 % (4 * RCX) == 0 && 256 % (4 * JV) == 0), "piece split");
+    uint4 pre[NJ];
+    auto fetch = [&](int t) {
+        const T* kv_t = kv + (int64_t)(k_at + t * KT) * ld_kv;
+        const T* ck_t = ck + (int64_t)(k_at + t * KT) * ld_ck + C;
+        const int left = nk - t * KT - 1;                     // rows past the last key repeat it (masked)
+        auto section = [&](auto per_row, auto count, int at, const T* base, int64_t ld) {
+            const int r0 = tid / per_row.value, c = tid % per_row.value;
 #pragma unroll
-        for (int j = 0; j < NPRE; ++j) {
-            int a, b, c;
-            pre[j] = piece(tid + 256 * j, 0, false, a, b, c);
-        }
-    }
+            for (int j = 0; j < count.value; ++j)
+                pre[at + j] = *reinterpret_cast<const uint4*>(base + (int64_t)min(r0 + j * (256 / per_row.value), left) * ld + 8 * c);
+        };
+        section(Int<4 * NKX>{}, Int<NKX>{}, 0, kv_t + (int64_t)h * N, ld_kv);
+        section(Int<4 * RCX>{}, Int<RCX>{}, NKX, ck_t, ld_ck);
+        section(Int<4 * JV>{}, Int<JV>{}, NKX + RCX, kv_t + (int64_t)H * N + (int64_t)h * V, ld_kv);
+    };
+    auto put = [&]() {
+        auto section = [&](auto per_row, auto count, int at, T* base, int ld) {
+            const int r0 = tid / per_row.value, c = tid % per_row.value;
+#pragma unroll
+            for (int j = 0; j < count.value; ++j)
+                *reinterpret_cast<uint4*>(base + (r0 + j * (256 / per_row.value)) * ld + 8 * c) = pre[at + j];
+        };
+        section(Int<4 * NKX>{}, Int<NKX>{}, 0, Ks, ldk);
+        section(Int<4 * RCX>{}, Int<RCX>{}, NKX, Ks + 32 * NKX, ldk);
+        section(Int<4 * JV>{}, Int<JV>{}, NKX + RCX, Vs, ldv);
+    };
+    if constexpr (EXACT) fetch(0);
     for (int t = 0; t < ntiles; ++t) {
         const int k0 = t * KT;
         if constexpr (EXACT) {
-#pragma unroll
-            for (int j = 0; j < NPRE; ++j) {
-                int a, b, c;
-                (void)piece(tid + 256 * j, t, true, a, b, c);
-                put(a, b, c, pre[j]);
-            }
+            put();
         } else {
             for (int p = tid; p < KT * ppr; p += 256) {
-                int a, b, c;
-                const uint4 v = piece(p, t, false, a, b, c);
-                put(a, b, c, v);
+                const int key = p / ppr;
+                int c = p - key * ppr;
+                const int64_t kk = k_at + min(k0 + key, nk - 1);
+                const T* src;
+                T* dst;
+                if (c < kn) {
+                    src = kv + kk * ld_kv + (int64_t)h * N + EPV * c;
+                    dst = Ks + key * ldk + EPV * c;
+                } else if (c < kn + kr) {
+                    c -= kn;
+                    src = ck + kk * ld_ck + C + EPV * c;
+                    dst = Ks + key * ldk + N + EPV * c;
+                } else {
+                    c -= kn + kr;
+                    src = kv + kk * ld_kv + (int64_t)H * N + (int64_t)h * V + EPV * c;
+                    dst = Vs + key * ldv + EPV * c;
+                }
+                *reinterpret_cast<uint4*>(dst) = *reinterpret_cast<const uint4*>(src);
             }
         }
         __syncthreads();
-        if constexpr (EXACT) {
-            if (t + 1 < ntiles) {
-#pragma unroll
-                for (int j = 0; j < NPRE; ++j) {
-                    int a, b, c;
-                    pre[j] = piece(tid + 256 * j, t + 1, false, a, b, c);
-                }
-            }
-        }
         f32x4 s[KT / 16][QT];
 #pragma unroll
         for (int kt = 0; kt < KT / 16; ++kt) {
@@ -488,22 +684,27 @@ __global__ __launch_bounds__(256, 1) void attn_prefill_kernel(const T* __restric
             mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
             mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
             mx = fmaxf(m_run[u], mx * scale);                 // (scale > 0; key 0 is visible to every row: finite from tile 0 on)
-            const float alpha = exp2f((m_run[u] - mx) * LOG2E), sc = scale * LOG2E, mb = mx * LOG2E;
+            const float alpha = __builtin_amdgcn_exp2f((m_run[u] - mx) * LOG2E), sc = scale * LOG2E, mb = mx * LOG2E;
             m_run[u] = mx;
             float sum = 0.f;
 #pragma unroll
             for (int kt = 0; kt < KT / 16; ++kt)
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
-                    const float p = exp2f(fmaf(s[kt][u][r], sc, -mb));
+                    const float p = __builtin_amdgcn_exp2f(fmaf(s[kt][u][r], sc, -mb));
                     sum += p;
                     pf[u][kt >> 1][(kt & 1) * 4 + r] = (T)p;
                 }
             l_run[u] = l_run[u] * alpha + sum;
+            if (!__all(alpha == 1.0f)) {                      // (most tiles leave every maximum where it was)
 #pragma unroll
-            for (int d = 0; d < DV; ++d)
+                for (int d = 0; d < DV; ++d)
 #pragma unroll
-                for (int r = 0; r < 4; ++r) o[u][d][r] *= alpha;
+                    for (int r = 0; r < 4; ++r) o[u][d][r] *= alpha;
+            }
+        }
+        if constexpr (EXACT) {                                // (here the score registers are free: two workgroups fit a CU)
+            if (t + 1 < ntiles) fetch(t + 1);
         }
 #pragma unroll
         for (int d = 0; d < DV; ++d) {
@@ -554,7 +755,7 @@ static int launch_prefill(const void* q, const void* kv, const void* ck, const i
         if (e != hipSuccess) return (int)e;
         attr = true;
     }
-    hipLaunchKernelGGL(k, dim3((max_new + 64 * QT - 1) / (64 * QT), H, nseq), dim3(256), lds, st, (const T*)q, (const T*)kv, (const T*)ck,
+    hipLaunchKernelGGL(k, dim3((max_new + 64 * QT - 1) / (64 * QT) * H, nseq), dim3(256), lds, st, (const T*)q, (const T*)kv, (const T*)ck,
                        seq, pos, cosb, sinb, half, max_pos, (const T*)gate, ld_gate, (T*)out, ld_out, tq, tk, H, N, R, V, C, scale);
     TFL_LAUNCH_CHECK();
     return TF_OK;

@@ -86,34 +86,37 @@ __device__ __forceinline__ float wave_sum64(float v) {
     for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
     return v;
 }
-// Sum over a 256-thread workgroup; red = 4 floats of LDS, free again after the call's second barrier.
-__device__ __forceinline__ float block_sum256(float v, float* red) {
+// Sum over a workgroup of NW waves; red = NW floats of LDS, free again after the call's second barrier.
+template <int NW> __device__ __forceinline__ float block_sum(float v, float* red) {
     v = wave_sum64(v);
     if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
     __syncthreads();
-    v = red[0] + red[1] + red[2] + red[3];
+    v = red[0];
+#pragma unroll
+    for (int w = 1; w < NW; ++w) v += red[w];
     __syncthreads();
     return v;
 }
 
-// One cache row from raw latent / key values: latent / rms(latent) * w, rotated key.  One 256-thread workgroup.
+// One cache row from raw latent / key values: latent / rms(latent) * w, rotated key.  One workgroup of NW waves.
 // src(c) reads raw element c of [latent C][key R].
-template <typename T, typename Src>
-__device__ __forceinline__ void cache_row_256(Src src, int C, int c_real, int R, const float* w, float eps, const float* cosr,
+template <typename T, int NW, typename Src>
+__device__ __forceinline__ void cache_row(Src src, int C, int c_real, int R, const float* w, float eps, const float* cosr,
                                               const float* sinr, int half, T* dst0, T* dst1, float* red) {
+    constexpr int NT = 64 * NW;
     float ss = 0.f;
-    for (int c = threadIdx.x; c < C; c += 256) {
+    for (int c = threadIdx.x; c < C; c += NT) {
         const float f = src(c);
         ss = fmaf(f, f, ss);
     }
-    ss = block_sum256(ss, red);
+    ss = block_sum<NW>(ss, red);
     const float inv = 1.0f / sqrtf(ss / (float)c_real + eps);
-    for (int c = threadIdx.x; c < C; c += 256) {
+    for (int c = threadIdx.x; c < C; c += NT) {
         const T o = (T)(src(c) * inv * w[c]);
         if (dst0) dst0[c] = o;
         if (dst1) dst1[c] = o;
     }
-    for (int p = threadIdx.x; p < R / 2; p += 256) {
+    for (int p = threadIdx.x; p < R / 2; p += NT) {
         float u = src(C + 2 * p), v = src(C + 2 * p + 1);
         if (p < half) {
             const float cs = cosr[p], sn = sinr[p], a = u * cs - v * sn;

@@ -12,35 +12,25 @@
 //   TOKEN     per-layer token input: gelu times the token's row of a table
 #include "latent_common.h"
 
-template <typename T, int XMODE>
-__device__ __forceinline__ typename El<T>::Frag load_x(const void* x, int64_t off, float inv, const float* nw) {
-    if constexpr (XMODE == TFL_X_T) {
-        return load_frag((const T*)x + off);
-    } else {
-        const f32x8 v = *reinterpret_cast<const f32x8*>((const float*)x + off);
-        typename El<T>::Frag f;
-        if constexpr (XMODE == TFL_X_F32_NORM) {
-            const f32x8 w = *reinterpret_cast<const f32x8*>(nw);
-#pragma unroll
-            for (int e = 0; e < 8; ++e) f[e] = (T)(v[e] * inv * w[e]);
-        } else {
-#pragma unroll
-            for (int e = 0; e < 8; ++e) f[e] = (T)v[e];
-        }
-        return f;
-    }
-}
+#ifndef TFL_PAIR_MIN
+#define TFL_PAIR_MIN 420     // panel pairs from which two panels share a workgroup
+#endif
 
-template <typename T, int XMODE, int EPI, int MT, int WAVES>
+template <typename T, int XMODE> struct RawX { typedef f32x8 Type; };
+template <typename T> struct RawX<T, TFL_X_T> { typedef typename El<T>::Frag Type; };
+
+// P panels per workgroup (they share the operand rows), MT 16-row blocks, U tiles of 32 per batch; AHEAD: the next batch's weights
+// are requested before the current one is used (long K), otherwise a wave's whole K range should fit one or two batches.
+template <typename T, int XMODE, int EPI, int P, int MT, int WAVES, int U, bool AHEAD>
 __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a) {
     typedef typename El<T>::Frag Frag;
-    constexpr int U = sizeof(T) == 2 ? 4 : 2;                // weight tiles in flight per wave and batch
-    __shared__ f32x4 part[WAVES][MT][64];
-    __shared__ float red[4];
+    typedef typename RawX<T, XMODE>::Type Raw;
+    static_assert(P * MT <= WAVES, "one wave finishes one 16x16 tile");
+    __shared__ f32x4 part[WAVES][P * MT][64];
     const int ppg = a.n >> 4, npan = ppg * a.groups;
     const int tid = threadIdx.x;
     if constexpr (EPI == TFL_EPI_QUERY) {
-        if ((int)blockIdx.x >= npan) {                       // cache row of batch row m (256-thread part of the workgroup)
+        if ((int)blockIdx.x >= npan) {                       // the cache row of one batch row
             const int m = blockIdx.y * (gridDim.x - npan) + blockIdx.x - npan;
             if (m >= a.rows) return;
             const int slot = a.slot[m];
@@ -48,71 +38,113 @@ __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a
             int p = a.pos[m];
             p = p < 0 ? 0 : (p >= a.max_pos ? a.max_pos - 1 : p);
             const float* src = a.kv_raw + (int64_t)m * a.ld_kv;
-            cache_row_256<T>([src](int c) { return src[c]; }, a.C, a.c_real, a.R, a.kv_norm_w, a.eps, a.cos + (int64_t)p * a.half,
-                             a.sin + (int64_t)p * a.half, a.half, (T*)a.cache + (int64_t)slot * (a.C + a.R), (T*)nullptr, red);
+            cache_row<T, WAVES>([src](int c) { return src[c]; }, a.C, a.c_real, a.R, a.kv_norm_w, a.eps, a.cos + (int64_t)p * a.half,
+                                a.sin + (int64_t)p * a.half, a.half, (T*)a.cache + (int64_t)slot * (a.C + a.R), (T*)nullptr,
+                                (float*)&part[0][0][0]);
             return;
         }
     }
     const int wave = tid >> 6, lane = tid & 63, g = lane >> 4, i = lane & 15;
-    const int panel = blockIdx.x, grp = panel / ppg, pin = panel - grp * ppg;
+    const int panel0 = blockIdx.x * P, grp = P == 1 ? panel0 / ppg : 0;
     const int m0 = blockIdx.y * 16 * MT;
     const int chunks = a.k >> 5;
     const int per = (chunks + WAVES - 1) / WAVES;
-    const int c_beg = wave * per, c_end = min(chunks, c_beg + per);
-    const T* wp = (const T*)a.wp + (int64_t)panel * chunks * 512 + lane * 8;
+    const int c_beg = wave * per, c_end = min(chunks, c_beg + per), last = c_end - 1;
+    const T* wp[P];
+#pragma unroll
+    for (int p = 0; p < P; ++p) wp[p] = (const T*)a.wp + (int64_t)min(panel0 + p, npan - 1) * chunks * 512 + lane * 8;
     int64_t xoff[MT];
-    float inv[MT];
+    int mrow[MT];
 #pragma unroll
     for (int t = 0; t < MT; ++t) {
-        const int m = min(m0 + 16 * t + i, a.rows - 1);
-        xoff[t] = (int64_t)m * a.ld_x + (int64_t)grp * a.x_group + 8 * g;
-        inv[t] = 1.f;
-        if constexpr (XMODE == TFL_X_F32_NORM) {             // the row's scale from the producer's per-panel sums of squares
-            float s = 0.f;
-            for (int p = g; p < a.ss_n; p += 4) s += a.ss_in[(int64_t)m * a.ss_ld + p];
-            s += __shfl_xor(s, 16, 64);
-            s += __shfl_xor(s, 32, 64);
-            inv[t] = 1.0f / sqrtf(s / (float)a.k_real + a.eps);
-        }
+        mrow[t] = min(m0 + 16 * t + i, a.rows - 1);
+        xoff[t] = (int64_t)mrow[t] * a.ld_x + (int64_t)grp * a.x_group + g * a.x_oct;
     }
-    f32x4 acc[MT];
+    const int64_t xstep = 4 * a.x_oct;
+    auto load_w = [&](Frag (&w)[P][U], int c0) {
 #pragma unroll
-    for (int t = 0; t < MT; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int u = 0; u < U; ++u)
+#pragma unroll
+            for (int p = 0; p < P; ++p) w[p][u] = load_frag_stream(wp[p] + (int64_t)min(c0 + u, last) * 512);
+    };
+    f32x4 acc[P][MT];
+#pragma unroll
+    for (int p = 0; p < P; ++p)
+#pragma unroll
+        for (int t = 0; t < MT; ++t) acc[p][t] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (c_beg < c_end) {
-        Frag w[U], wn[U];
-        const int last = c_end - 1;
-#pragma unroll
-        for (int u = 0; u < U; ++u) w[u] = load_frag_stream(wp + (int64_t)min(c_beg + u, last) * 512);
+        float inv[MT];
+        bool scaled = false;
+        Frag w[P][U], wn[P][U];
+        load_w(w, c_beg);
         for (int c0 = c_beg; c0 < c_end; c0 += U) {
-            Frag xv[U][MT];
+            Raw xr[U][MT];
+            f32x8 nw[U];
 #pragma unroll
             for (int u = 0; u < U; ++u) {
                 const int c = min(c0 + u, last);
 #pragma unroll
-                for (int t = 0; t < MT; ++t)
-                    xv[u][t] = load_x<T, XMODE>(a.x, xoff[t] + 32 * (int64_t)c, inv[t], (const float*)a.norm_w + 32 * c + 8 * g);
+                for (int t = 0; t < MT; ++t) {
+                    if constexpr (XMODE == TFL_X_T) xr[u][t] = load_frag((const T*)a.x + xoff[t] + xstep * c);
+                    else xr[u][t] = *reinterpret_cast<const f32x8*>((const float*)a.x + xoff[t] + xstep * c);
+                }
+                if constexpr (XMODE == TFL_X_F32_NORM) nw[u] = *reinterpret_cast<const f32x8*>((const float*)a.norm_w + 32 * c + 8 * g);
             }
+            if constexpr (AHEAD) load_w(wn, c0 + U);
+            if constexpr (XMODE == TFL_X_F32_NORM) {         // the row's scale from the producer's per-panel sums of squares
+                if (!scaled) {
 #pragma unroll
-            for (int u = 0; u < U; ++u) wn[u] = load_frag_stream(wp + (int64_t)min(c0 + U + u, last) * 512);
+                    for (int t = 0; t < MT; ++t) {
+                        float s = 0.f;
+#pragma unroll 4
+                        for (int p = g; p < a.ss_n; p += 4) s += a.ss_in[(int64_t)mrow[t] * a.ss_ld + p];
+                        s += __shfl_xor(s, 16, 64);
+                        s += __shfl_xor(s, 32, 64);
+                        inv[t] = 1.0f / sqrtf(s / (float)a.k_real + a.eps);
+                    }
+                    scaled = true;
+                }
+            }
 #pragma unroll
             for (int u = 0; u < U; ++u)
                 if (c0 + u < c_end) {
 #pragma unroll
-                    for (int t = 0; t < MT; ++t) acc[t] = El<T>::mma(w[u], xv[u][t], acc[t]);
-                }
+                    for (int t = 0; t < MT; ++t) {
+                        Frag x;
+                        if constexpr (XMODE == TFL_X_T) x = xr[u][t];
+                        else {
 #pragma unroll
-            for (int u = 0; u < U; ++u) w[u] = wn[u];
+                            for (int e = 0; e < 8; ++e) {
+                                if constexpr (XMODE == TFL_X_F32_NORM) x[e] = (T)(xr[u][t][e] * inv[t] * nw[u][e]);
+                                else x[e] = (T)xr[u][t][e];
+                            }
+                        }
+#pragma unroll
+                        for (int p = 0; p < P; ++p) acc[p][t] = El<T>::mma(w[p][u], x, acc[p][t]);
+                    }
+                }
+            if constexpr (AHEAD) {
+#pragma unroll
+                for (int p = 0; p < P; ++p)
+#pragma unroll
+                    for (int u = 0; u < U; ++u) w[p][u] = wn[p][u];
+            } else if (c0 + U < c_end) {
+                load_w(w, c0 + U);
+            }
         }
     }
 #pragma unroll
-    for (int t = 0; t < MT; ++t) part[wave][t][lane] = acc[t];
+    for (int p = 0; p < P; ++p)
+#pragma unroll
+        for (int t = 0; t < MT; ++t) part[wave][p * MT + t][lane] = acc[p][t];
     __syncthreads();
-    if (wave >= MT) return;                                  // wave t finishes row block t
-    const int t = wave;
-    f32x4 s = part[0][t][lane];
+    if (wave >= P * MT) return;                              // wave p * MT + t finishes row block t of panel p
+    const int t = wave % MT, panel = panel0 + wave / MT, pin = P == 1 ? panel - grp * ppg : panel;
+    if (panel >= npan) return;
+    f32x4 s = part[0][wave][lane];
 #pragma unroll
     for (int w = 1; w < WAVES; ++w) {
-        const f32x4 o = part[w][t][lane];
+        const f32x4 o = part[w][wave][lane];
 #pragma unroll
         for (int r = 0; r < 4; ++r) s[r] += o[r];
     }
@@ -131,7 +163,8 @@ __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a
         } else if (live) {
 #pragma unroll
             for (int r = 0; r < 4; ++r) s[r] = gelu_tanh(s[r]);
-            store_quad((T*)a.out_t + (int64_t)m * a.ld_t + (n - a.n_raw), s);
+            const int k = n - a.n_raw;
+            store_quad((T*)a.out_t + (int64_t)m * a.ld_t + (k >> 3) * a.t_oct + (k & 7), s);
         }
         return;
     }
@@ -169,7 +202,7 @@ __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a
         const f32x4 z = *reinterpret_cast<const f32x4*>(a.gate + (int64_t)m * a.ld_gate + col);
 #pragma unroll
         for (int r = 0; r < 4; ++r) s[r] *= sigmoid(z[r]);
-        store_quad((T*)a.out_t + (int64_t)m * a.ld_t + col, s);
+        store_quad((T*)a.out_t + (int64_t)m * a.ld_t + (col >> 3) * a.t_oct + (col & 7), s);
     } else if constexpr (EPI == TFL_EPI_RESIDUAL) {
         f32x4* y = reinterpret_cast<f32x4*>(a.out_f + (int64_t)m * a.ld_f + n);
         f32x4 o = *y;
@@ -186,27 +219,39 @@ __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a
     }
 }
 
+template <typename T, int XMODE, int EPI, int P, int WAVES, int U, bool AHEAD>
+static int launch_form(const TflGemm& a, hipStream_t st) {
+    const int panels = (a.n >> 4) * a.groups;
+    const int mt = a.rows <= 16 ? 1 : 2, rb = (a.rows + 16 * mt - 1) / (16 * mt);
+    const int extra = EPI == TFL_EPI_QUERY && a.kv_raw ? (a.rows + rb - 1) / rb : 0;
+    const dim3 grid((panels + P - 1) / P + extra, rb), block(64 * WAVES);
+    if (mt == 1) hipLaunchKernelGGL((latent_gemm_kernel<T, XMODE, EPI, P, 1, WAVES, U, AHEAD>), grid, block, 0, st, a);
+    else hipLaunchKernelGGL((latent_gemm_kernel<T, XMODE, EPI, P, 2, WAVES, U, AHEAD>), grid, block, 0, st, a);
+    TFL_LAUNCH_CHECK();
+    return TF_OK;
+}
+
+// Waves per panel by panel count (few panels: more waves keep the weight stream deep enough); wide outputs take two panels per
+// workgroup.  The small per-head / latent products issue a wave's whole K range at once.
 template <typename T, int XMODE, int EPI>
 static int launch_gemm(const TflGemm& a, hipStream_t st) {
     const int panels = (a.n >> 4) * a.groups;
-    const int mt = a.rows <= 16 ? 1 : 2;
-    const int rb = (a.rows + 16 * mt - 1) / (16 * mt);
-    int extra = 0;
-    if (EPI == TFL_EPI_QUERY && a.kv_raw) extra = (a.rows + rb - 1) / rb;
-    const dim3 grid(panels + extra, rb);
-    // few panels: more waves per panel keep the weight stream deep enough; the cache-row workgroups are written for 4 waves
-    if (EPI == TFL_EPI_QUERY || panels > 1024) {
-        if (mt == 1) hipLaunchKernelGGL((latent_gemm_kernel<T, XMODE, EPI, 1, 4>), grid, dim3(256), 0, st, a);
-        else hipLaunchKernelGGL((latent_gemm_kernel<T, XMODE, EPI, 2, 4>), grid, dim3(256), 0, st, a);
-    } else if (panels > 128) {
-        if (mt == 1) hipLaunchKernelGGL((latent_gemm_kernel<T, XMODE, EPI, 1, 8>), grid, dim3(512), 0, st, a);
-        else hipLaunchKernelGGL((latent_gemm_kernel<T, XMODE, EPI, 2, 8>), grid, dim3(512), 0, st, a);
+    if constexpr (sizeof(T) == 4) {
+        return launch_form<T, XMODE, EPI, 1, 8, 2, true>(a, st);
+    } else if constexpr (EPI == TFL_EPI_IN || EPI == TFL_EPI_F32 || EPI == TFL_EPI_RESIDUAL) {
+        if (panels >= 2 * TFL_PAIR_MIN) return launch_form<T, XMODE, EPI, 2, 4, 4, true>(a, st);
+        if (panels > 512) return launch_form<T, XMODE, EPI, 1, 4, 4, true>(a, st);
+        if (panels > 128) return launch_form<T, XMODE, EPI, 1, 8, 4, true>(a, st);
+        return launch_form<T, XMODE, EPI, 1, 16, 4, true>(a, st);
+    } else if constexpr (XMODE != TFL_X_T) {                  // (fp32 operands: registers for half the batch)
+        if (panels > 512) return launch_form<T, XMODE, EPI, 1, 4, 4, true>(a, st);
+        if (panels > 128 || EPI == TFL_EPI_QUERY) return launch_form<T, XMODE, EPI, 1, 8, 4, true>(a, st);
+        return launch_form<T, XMODE, EPI, 1, 16, 4, true>(a, st);
     } else {
-        if (mt == 1) hipLaunchKernelGGL((latent_gemm_kernel<T, XMODE, EPI, 1, 16>), grid, dim3(1024), 0, st, a);
-        else hipLaunchKernelGGL((latent_gemm_kernel<T, XMODE, EPI, 2, 16>), grid, dim3(1024), 0, st, a);
+        if (panels > 512) return launch_form<T, XMODE, EPI, 1, 4, 8, false>(a, st);
+        if (panels > 128) return launch_form<T, XMODE, EPI, 1, 8, 8, false>(a, st);
+        return launch_form<T, XMODE, EPI, 1, 16, 8, false>(a, st);
     }
-    TFL_LAUNCH_CHECK();
-    return TF_OK;
 }
 
 template <typename T>
@@ -227,7 +272,8 @@ extern "C" int tfl_gemm(const TflGemm* p, int dtype, int x_mode, int epi, void* 
     if (!p || !p->wp || !p->x) return TF_EINVAL;
     const TflGemm a = *p;
     if (a.rows < 1 || a.rows > (1 << 20) || a.n < 16 || (a.n & 15) || a.k < 32 || (a.k & 31) || a.groups < 1) return TF_EINVAL;
-    if (a.ld_x & 7 || a.x_group & 7) return TF_EINVAL;
+    if ((a.ld_x & 7) || (a.x_group & 7) || a.x_oct < 8 || (a.x_oct & 7) || a.ld_x < 8) return TF_EINVAL;
+    if (a.out_t && (a.t_oct < 8 || (a.t_oct & 7))) return TF_EINVAL;
     if (dtype != 0 && dtype != 1) return TF_EINVAL;
     switch (epi) {
         case TFL_EPI_F32:
@@ -236,7 +282,7 @@ extern "C" int tfl_gemm(const TflGemm* p, int dtype, int x_mode, int epi, void* 
         case TFL_EPI_IN:
             if (!a.out_f || !a.ss_out || a.groups != 1 || a.n_raw < 16 || (a.n_raw & 15) || a.n_raw > a.n || a.ld_f < a.n_raw
                 || (a.ld_f & 3) || a.ss_ld < a.n_raw / 16) return TF_EINVAL;
-            if (a.n_raw < a.n && (!a.out_t || (a.ld_t & 3) || a.ld_t < a.n - a.n_raw)) return TF_EINVAL;
+            if (a.n_raw < a.n && (!a.out_t || (a.ld_t & 7) || a.ld_t < 8)) return TF_EINVAL;
             break;
         case TFL_EPI_QUERY:
             if (!a.out_t || !a.out_t2 || !a.pos || a.groups != 1 || a.H < 1 || a.N < 16 || a.R < 0 || a.C < 16) return TF_EINVAL;
@@ -250,8 +296,7 @@ extern "C" int tfl_gemm(const TflGemm* p, int dtype, int x_mode, int epi, void* 
             if (!a.out_t || a.groups != a.H || a.C != a.n || a.R < 0 || (a.R & 3)) return TF_EINVAL;
             break;
         case TFL_EPI_GATED:
-            if (!a.out_t || !a.gate || a.ld_t < (int64_t)a.groups * a.n || a.ld_gate < (int64_t)a.groups * a.n || (a.ld_t & 3)
-                || (a.ld_gate & 3)) return TF_EINVAL;
+            if (!a.out_t || !a.gate || a.ld_t < 8 || a.ld_gate < (int64_t)a.groups * a.n || (a.ld_t & 7) || (a.ld_gate & 3)) return TF_EINVAL;
             break;
         case TFL_EPI_RESIDUAL:
             if (!a.out_f || a.groups != 1 || a.ld_f < a.n || (a.ld_f & 3)) return TF_EINVAL;

@@ -8,8 +8,8 @@ template <typename T, typename Y>
 __global__ __launch_bounds__(256) void finish_kernel(const T* __restrict__ embed, const int64_t* __restrict__ ids, int vocab,
                                                      const Y* __restrict__ y, int64_t ld_y, const float* __restrict__ y_w,
                                                      const float* __restrict__ step, const float* __restrict__ norm_w,
-                                                     float* __restrict__ x, T* __restrict__ h, int width, int width_real,
-                                                     float eps) {
+                                                     float* __restrict__ x, T* __restrict__ h, int64_t ld_h, int64_t h_oct,
+                                                     int width, int width_real, float eps) {
     __shared__ float red[4];
     const int row = blockIdx.x, nq = width >> 2;             // elements in groups of 4
     float* xr = x + (int64_t)row * width;
@@ -27,7 +27,7 @@ __global__ __launch_bounds__(256) void finish_kernel(const T* __restrict__ embed
             const f32x4 v = load_quad(yr + 4 * q);
             s += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
         }
-        s = block_sum256(s, red);
+        s = block_sum<4>(s, red);
         yi = 1.0f / sqrtf(s / (float)width_real + eps);
     }
     float s = 0.f;
@@ -46,26 +46,26 @@ __global__ __launch_bounds__(256) void finish_kernel(const T* __restrict__ embed
         s += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
         if (er || yr || step) *reinterpret_cast<f32x4*>(xr + 4 * q) = v;
     }
-    s = block_sum256(s, red);
+    s = block_sum<4>(s, red);
     const float inv = 1.0f / sqrtf(s / (float)width_real + eps);
     for (int q = threadIdx.x; q < nq; q += 256) {             // (each thread re-reads what it wrote itself)
         f32x4 v = *reinterpret_cast<const f32x4*>(xr + 4 * q);
         const f32x4 w = *reinterpret_cast<const f32x4*>(norm_w + 4 * q);
 #pragma unroll
         for (int r = 0; r < 4; ++r) v[r] = v[r] * inv * w[r];
-        store_quad(h + (int64_t)row * width + 4 * q, v);
+        store_quad(h + (int64_t)row * ld_h + (q >> 1) * h_oct + 4 * (q & 1), v);
     }
 }
 
 extern "C" int tfl_finish(const void* embed, const int64_t* ids, int vocab, const void* y, int y_f32, int64_t ld_y,
-                          const float* y_w, const float* step, const float* norm_w, float* x, void* h, int rows, int width,
-                          int width_real, float eps, int dtype, void* stream) {
-    if (!x || !h || !norm_w || rows < 1 || width < 4 || (width & 3) || width_real < 1 || width_real > width) return TF_EINVAL;
+                          const float* y_w, const float* step, const float* norm_w, float* x, void* h, int64_t ld_h, int64_t h_oct,
+                          int rows, int width, int width_real, float eps, int dtype, void* stream) {
+    if (!x || !h || !norm_w || rows < 1 || width < 8 || (width & 7) || ld_h < 8 || (ld_h & 7) || h_oct < 8 || (h_oct & 7) || width_real < 1 || width_real > width) return TF_EINVAL;
     if (embed && (!ids || vocab < 1)) return TF_EINVAL;
     if (y && (!y_w || ld_y < width || (ld_y & 3))) return TF_EINVAL;
     hipStream_t st = (hipStream_t)stream;
 #define GO(T, Y) hipLaunchKernelGGL((finish_kernel<T, Y>), dim3(rows), dim3(256), 0, st, (const T*)embed, ids, vocab, (const Y*)y, \
-                                    ld_y, y_w, step, norm_w, x, (T*)h, width, width_real, eps)
+                                    ld_y, y_w, step, norm_w, x, (T*)h, ld_h, h_oct, width, width_real, eps)
     if (dtype == 0) { if (y_f32) GO(bf16, float); else GO(bf16, bf16); }
     else if (dtype == 1) GO(float, float);
     else return TF_EINVAL;
@@ -142,7 +142,7 @@ __global__ __launch_bounds__(256) void prepare_kernel(const T* __restrict__ y, i
         const f32x4 v = load_quad(yr + 4 * c);
         s += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
     }
-    s = block_sum256(s, red);
+    s = block_sum<4>(s, red);
     const float inv = 1.0f / sqrtf(s / (float)q_real + eps);
     for (int c = threadIdx.x; c < q / 4; c += 256) {
         f32x4 v = load_quad(yr + 4 * c);
@@ -155,7 +155,7 @@ __global__ __launch_bounds__(256) void prepare_kernel(const T* __restrict__ y, i
     p = p < 0 ? 0 : (p >= max_pos ? max_pos - 1 : p);
     const int sl = slot[row], W = C + R;
     const T* kv = yr + q;
-    cache_row_256<T>([kv](int c) { return (float)kv[c]; }, C, c_real, R, kv_norm, eps, cosb + (int64_t)p * half,
+    cache_row<T, 4>([kv](int c) { return (float)kv[c]; }, C, c_real, R, kv_norm, eps, cosb + (int64_t)p * half,
                      sinb + (int64_t)p * half, half, sl >= 0 && sl < cache_rows ? cache + (int64_t)sl * W : (T*)nullptr,
                      ck ? ck + (int64_t)row * W : (T*)nullptr, red);
     for (int c = threadIdx.x; c < n_up / 4; c += 256) {

@@ -108,7 +108,7 @@ class LatentLayer:
     # -- the two forms of a layer: h (normed input), x (fp32 residual, updated) -> y (token-side output, added by the next norm) ----
     def decode(self, h, x, ids, side_table, batch, rope, cache_rows, eps):
         g = self.geom
-        act = torch.empty(h.shape[0], self.w_out.k, dtype=h.dtype, device=h.device)
+        act = ol.empty_act(ids.numel(), self.w_out.k, h.dtype, h.device)
         raw, ss = ol.input_projection(h, self.w_in, g.n_raw, act, g.H * g.V)
         qn, q = ol.query_and_append(raw, ss, self.w_uq, g, self.q_norm, self.kv_norm, eps, rope, batch.pos, batch.slot, cache_rows)
         ol.query_to_latent(qn, self.w_uk_t, q, g)

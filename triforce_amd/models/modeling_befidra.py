@@ -86,7 +86,7 @@ class BefidraForCausalLM:
         for r, (i, t, first) in enumerate(self.runs):
             L = W.layers[i]
             h = ol.finish(x, L.norm1, eps, width, self.dtype, embed=W.embed if r == 0 else None, ids=ids if r == 0 else None,
-                          y=y, y_w=y_w, step=W.step[t] if first else None)
+                          y=y, y_w=y_w, step=W.step[t] if first else None, octets=batch.decode)
             if W.capture is not None and r > 0:
                 W.capture.append((x - W.step[t] if first else x.clone())[:, :width])
             layer = L.decode if batch.decode else L.prefill

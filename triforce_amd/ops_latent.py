@@ -72,10 +72,34 @@ class TileWeight:
         return F.linear(x, self.w)
 
 
+def empty_act(rows, k, dtype, device):
+    """Octet-major activation block [k/8, rows, 8] (include/triforce_latent.h); a 2-D tensor is a row-major one."""
+    return torch.empty(k // 8, rows, 8, dtype=dtype, device=device)
+
+
+def act_rows(x):
+    """Row-major copy of an activation block."""
+    return x if x.dim() == 2 else x.permute(1, 0, 2).reshape(x.shape[1], -1)
+
+
+def _lay(x):
+    """(rows, k, ld, oct) of an activation block."""
+    if x.dim() == 3:
+        assert x.shape[2] == 8 and x.is_contiguous()
+        return x.shape[1], 8 * x.shape[0], 8, 8 * x.shape[1]
+    return x.shape[0], x.shape[1], x.stride(0), 8
+
+
+def _tail(x, k):
+    """The columns from k on."""
+    return x[k // 8:] if x.dim() == 3 else x[:, k:]
+
+
 def _gemm(wt, x, x_mode, epi, rows, **kw):
     a = hip.TflGemm()
     a.wp, a.x = wt.packed.data_ptr(), x.data_ptr()
     a.rows, a.n, a.k, a.groups = rows, wt.n, wt.k, wt.groups
+    a.x_oct = a.t_oct = 8
     for name, v in kw.items():
         setattr(a, name, v.data_ptr() if isinstance(v, torch.Tensor) else v)
     hip.check(hip.latent_lib().tfl_gemm(ctypes.byref(a), _CODE[wt.dtype], hip.TFL_X[x_mode], hip.TFL_EPI[epi], _stream()), "tfl_gemm " + epi)
@@ -84,26 +108,27 @@ def _gemm(wt, x, x_mode, epi, rows, **kw):
 def linear_f32(x, wt, n_real, out=None):
     """fp32 x . W^T (logits, the token-side projection): x [rows, k] of the weight's type."""
     _need(x)
-    rows = x.shape[0]
-    assert x.dtype == wt.dtype and x.shape[1] == wt.k
+    rows, k, ld, octet = _lay(x)
+    assert x.dtype == wt.dtype and k == wt.k
     if out is None:
         out = torch.empty(rows, n_real, dtype=torch.float32, device=x.device)
     assert out.dtype == torch.float32 and out.shape[0] == rows and out.shape[1] >= n_real and out.stride(1) == 1
-    _gemm(wt, x, "t", "f32", rows, ld_x=x.stride(0), out_f=out, ld_f=out.stride(0), n_real=n_real)
+    _gemm(wt, x, "t", "f32", rows, ld_x=ld, x_oct=octet, out_f=out, ld_f=out.stride(0), n_real=n_real)
     return out
 
 
 def input_projection(h, wt, n_raw, act, act_off):
-    """All projections of the layer's one norm.  Returns (raw fp32 [rows, n_raw], per-panel sums of squares); gelu of the other
-    outputs goes to act[:, act_off:]."""
+    """All projections of the layer's one norm (h, act: activation blocks).  Returns (raw fp32 [rows, n_raw], per-panel sums of
+    squares); gelu of the other outputs goes to the columns of act from act_off on."""
     _need(h, act)
-    rows = h.shape[0]
-    assert h.dtype == wt.dtype == act.dtype and h.shape[1] == wt.k and act.shape[1] >= act_off + wt.n - n_raw
+    rows, k, ld, octet = _lay(h)
+    act_rows_, act_k, act_ld, act_oct = _lay(act)
+    assert h.dtype == wt.dtype == act.dtype and k == wt.k and act_rows_ == rows and act_k >= act_off + wt.n - n_raw and act_off % 8 == 0
     raw = torch.empty(rows, n_raw, dtype=torch.float32, device=h.device)
     ss = torch.empty(rows, n_raw // 16, dtype=torch.float32, device=h.device)
-    tail = act[:, act_off:] if wt.n > n_raw else act
-    _gemm(wt, h, "t", "in", rows, ld_x=h.stride(0), out_f=raw, ld_f=n_raw, ss_out=ss, ss_ld=n_raw // 16, n_raw=n_raw,
-          out_t=tail, ld_t=act.stride(0))
+    tail = _tail(act, act_off) if wt.n > n_raw else act
+    _gemm(wt, h, "t", "in", rows, ld_x=ld, x_oct=octet, out_f=raw, ld_f=n_raw, ss_out=ss, ss_ld=n_raw // 16, n_raw=n_raw,
+          out_t=tail, ld_t=act_ld, t_oct=act_oct)
     return raw, ss
 
 
@@ -137,21 +162,22 @@ def query_to_latent(qn, wt, q, g):
 
 
 def latent_to_value(ol, wt, raw, gate_off, act, g):
-    """act[:, h*V:(h+1)*V] = (ol[:, h] . Wuv_h^T) * sigmoid(gate)."""
+    """Columns h*V .. of the activation block act = (ol[:, h] . Wuv_h^T) * sigmoid(gate)."""
     _need(ol, raw, act)
-    rows = ol.shape[0]
-    assert (wt.groups, wt.n, wt.k) == (g.H, g.V, g.C) and ol.dtype == act.dtype == wt.dtype and act.shape[1] >= g.H * g.V
+    rows, (act_rows_, act_k, act_ld, act_oct) = ol.shape[0], _lay(act)
+    assert (wt.groups, wt.n, wt.k) == (g.H, g.V, g.C) and ol.dtype == act.dtype == wt.dtype and act_rows_ == rows and act_k >= g.H * g.V
     assert raw.shape[1] >= gate_off + g.H * g.V
     _gemm(wt, ol, "t", "gated", rows, ld_x=g.H * g.C, x_group=g.C, gate=raw[:, gate_off:], ld_gate=raw.stride(0), out_t=act,
-          ld_t=act.stride(0))
+          ld_t=act_ld, t_oct=act_oct)
 
 
 def add_linear(act, wt, x):
     """x (fp32) += act . W^T."""
     _need(act, x)
     _f32(x)
-    assert act.dtype == wt.dtype and act.shape[1] == wt.k and x.shape == (act.shape[0], wt.n) and x.is_contiguous()
-    _gemm(wt, act, "t", "residual", act.shape[0], ld_x=act.stride(0), out_f=x, ld_f=x.stride(0))
+    rows, k, ld, octet = _lay(act)
+    assert act.dtype == wt.dtype and k == wt.k and x.shape == (rows, wt.n) and x.is_contiguous()
+    _gemm(wt, act, "t", "residual", rows, ld_x=ld, x_oct=octet, out_f=x, ld_f=x.stride(0))
 
 
 def token_gate_linear(x, wt, table, ids, n_real):
@@ -165,9 +191,9 @@ def token_gate_linear(x, wt, table, ids, n_real):
     return out
 
 
-def finish(x, norm_w, eps, width, dtype, embed=None, ids=None, y=None, y_w=None, step=None):
+def finish(x, norm_w, eps, width, dtype, embed=None, ids=None, y=None, y_w=None, step=None, octets=False):
     """Residual bookkeeping between two layers and the next norm; see tfl_finish.  x fp32 [rows, padded width] is updated in
-    place; returns h in ``dtype``."""
+    place; returns h in ``dtype``, row-major or (``octets``) octet-major."""
     _need(x, norm_w, embed, ids, y, y_w, step)
     _f32(x, norm_w, y_w, step)
     rows, wp = x.shape
@@ -175,10 +201,11 @@ def finish(x, norm_w, eps, width, dtype, embed=None, ids=None, y=None, y_w=None,
     assert embed is None or (embed.dtype == dtype and embed.shape[1] == wp and embed.is_contiguous() and ids.numel() == rows
                              and ids.dtype == torch.int64)
     assert y is None or (y.shape == (rows, wp) and y_w.numel() == wp and y.dtype in (dtype, torch.float32) and y.stride(1) == 1)
-    h = torch.empty(rows, wp, dtype=dtype, device=x.device)
+    h = empty_act(rows, wp, dtype, x.device) if octets else torch.empty(rows, wp, dtype=dtype, device=x.device)
+    _, _, ld, octet = _lay(h)
     hip.check(hip.latent_lib().tfl_finish(_p(embed), _p(ids), 0 if embed is None else embed.shape[0], _p(y),
                                           int(y is not None and y.dtype == torch.float32), 0 if y is None else y.stride(0), _p(y_w),
-                                          _p(step), _p(norm_w), _p(x), _p(h), rows, wp, width, float(eps), _CODE[dtype], _stream()),
+                                          _p(step), _p(norm_w), _p(x), _p(h), ld, octet, rows, wp, width, float(eps), _CODE[dtype], _stream()),
               "tfl_finish")
     return h
 

@@ -79,11 +79,12 @@ def befidra_decode_kernels(m, rows, ctx):
     h = torch.randn(W.layers[0].width // 8, rows, 8, device=dev).to(m.dtype)
     x, ids = torch.randn(rows, WIDTH, device=dev), torch.arange(rows, device=dev)
     act = torch.randn(W.layers[0].w_out.k // 8, rows, 8, device=dev).to(m.dtype)
-    raw, ss = ol.input_projection(h, W.layers[0].w_in, g.n_raw, act, g.H * g.V)
-    qn, q = ol.query_and_append(raw, ss, W.layers[0].w_uq, g, W.layers[0].q_norm, W.layers[0].kv_norm, 1e-5, rope, pos, slot, cache.rows[0])
+    raw, ss, xq = ol.input_projection(h, W.layers[0].w_in, g.n_raw, W.layers[0].q_norm, act, g.H * g.V)
+    qn, q = ol.query_and_append(xq, raw, ss, W.layers[0].w_uq, g, W.layers[0].kv_norm, 1e-5, rope, pos, slot, cache.rows[0])
     o = torch.randn(rows, g.H, g.C, device=dev).to(m.dtype)
     side = W.side_table(0)
-    sg = ol.token_gate_linear(x, W.layers[0].side_gate, side, ids, 256)
+    xt = ol.add_linear(act, W.layers[0].w_out, x, True)
+    sg = ol.token_gate_linear(xt, W.layers[0].side_gate, side, ids, 256)
     y = ol.linear_f32(sg, W.layers[0].side_proj, WIDTH)
 
     def wb(w):
@@ -93,17 +94,17 @@ def befidra_decode_kernels(m, rows, ctx):
     out = [
         _kernel(R, "befidra", "finish (norm)", [lambda: ol.finish(x, k0.norm1, 1e-5, WIDTH, m.dtype, y=y, y_w=k0.side_norm, octets=True)] * 4,
                 R * WIDTH * 14, like="rmsnorm"),
-        _kernel(R, "befidra", "input projections", [lambda l=l: ol.input_projection(h, l.w_in, g.n_raw, act, g.H * g.V) for l in L],
+        _kernel(R, "befidra", "input projections", [lambda l=l: ol.input_projection(h, l.w_in, g.n_raw, l.q_norm, act, g.H * g.V) for l in L],
                 wb(k0.w_in), 2.0 * R * k0.w_in.n * k0.w_in.k, like="gate|up"),
         _kernel(R, "befidra", "query up + cache append",
-                [lambda l=l: ol.query_and_append(raw, ss, l.w_uq, g, l.q_norm, l.kv_norm, 1e-5, rope, pos, slot, cache.rows[0]) for l in L],
+                [lambda l=l: ol.query_and_append(xq, raw, ss, l.w_uq, g, l.kv_norm, 1e-5, rope, pos, slot, cache.rows[0]) for l in L],
                 wb(k0.w_uq), like="o"),
         _kernel(R, "befidra", "query to latent", [lambda l=l: ol.query_to_latent(qn, l.w_uk_t, q, g) for l in L], wb(k0.w_uk_t)),
         _kernel(R, "befidra", "latent to value + gate", [lambda l=l: ol.latent_to_value(o, l.w_uv, raw, g.gate_off, act, g) for l in L],
                 wb(k0.w_uv)),
-        _kernel(R, "befidra", "output + down", [lambda l=l: ol.add_linear(act, l.w_out, x) for l in L], wb(k0.w_out),
+        _kernel(R, "befidra", "output + down", [lambda l=l: ol.add_linear(act, l.w_out, x, True) for l in L], wb(k0.w_out),
                 2.0 * R * k0.w_out.n * k0.w_out.k, like="down"),
-        _kernel(R, "befidra", "token gate", [lambda l=l: ol.token_gate_linear(x, l.side_gate, side, ids, 256) for l in L], wb(k0.side_gate)),
+        _kernel(R, "befidra", "token gate", [lambda l=l: ol.token_gate_linear(xt, l.side_gate, side, ids, 256) for l in L], wb(k0.side_gate)),
         _kernel(R, "befidra", "token projection", [lambda l=l: ol.linear_f32(sg, l.side_proj, WIDTH) for l in L], wb(k0.side_proj)),
         _kernel(R, "befidra", "logits", [lambda: ol.linear_f32(h, W.logits, m.vocab_size)] * 2, wb(W.logits), like="lm_head"),
         _kernel(R, "befidra", "attention (+ merge)",
@@ -256,7 +257,7 @@ def run_design(args):
     with torch.inference_mode():
         for r, ctx in ((1, 32768), (8, 4096), (8, 32768), (32, 4096)):
             befidra_decode_kernels(bm, r, ctx)
-        for r, ctx in ((1, 32768), (8, 32768), (32, 4096), (1, 124928)):
+        for r, ctx in ((1, 2304), (1, 32768), (8, 4096), (8, 32768), (32, 4096), (1, 124928)):
             llama_decode_kernels(lm, r, ctx)
         for new, past in ((4096, 0), (4096, 28672)):
             prefill_kernels(bm, lm, new, past)

@@ -35,21 +35,19 @@ int tfl_abi_version(void);
 enum {
     TFL_EPI_F32 = 0,                /* out_f[m*ld_f + n] = acc, n < n_real */
     TFL_EPI_IN = 1,                 /* n < n_raw: out_f[m*ld_f + n] = acc and ss[m*(n_raw/16) + n/16] = sum over the panel of
-                                       acc^2; else out_t(m, n - n_raw) = gelu_tanh(acc) */
-    TFL_EPI_QUERY = 2,              /* heads of N + R outputs: out_t2[(m*H + h)*N + n] unrotated;
+                                       acc^2, and for n < n_scaled out_t2 = acc * norm_w[n]
+                                       (octet-major); else out_t(m, n - n_raw) = gelu_tanh(acc) */
+    TFL_EPI_QUERY = 2,              /* acc *= 1 / sqrt(sum(ss_in[m][:ss_n]) / k_real + eps); heads of N + R outputs: out_t2[(m*H + h)*N + n] unrotated;
                                        out_t[(m*H + h)*(C + R) + C + n] rotated at pos[m] */
     TFL_EPI_LATENT = 3,             /* group h: out_t[(m*H + h)*(C + R) + n] = acc */
     TFL_EPI_GATED = 4,              /* group h: out_t(m, h*ppg*16 + n) = acc * sigmoid(gate[m*ld_gate + h*ppg*16 + n]) */
-    TFL_EPI_RESIDUAL = 5,           /* out_f[m*ld_f + n] += acc */
+    TFL_EPI_RESIDUAL = 5,           /* out_f[m*ld_f + n] += acc; out_t(m, n) = the sum when out_t is given */
     TFL_EPI_TOKEN = 6               /* out_t[m*ld_t + n] = gelu_tanh(acc) * tok_table[ids[m]*ld_tok + n], n < n_real (0 behind) */
 };
-/* Where the GEMM's rows come from. */
-enum { TFL_X_T = 0, TFL_X_F32 = 1, TFL_X_F32_NORM = 2 };   /* _NORM: x * rsqrt(sum(ss[m][:])/k_real + eps) * norm_w */
-
 typedef struct TflGemm {
     const void* wp;                 /* packed weights, groups back to back */
     const void* x;
-    const void* norm_w;             /* fp32 [k] (TFL_X_F32_NORM) */
+    const float* norm_w;            /* [n_scaled] */
     const float* ss_in;             /* [rows][ss_n]: the first ss_n panels' sums of squares, row stride ss_ld */
     void* out_t;
     void* out_t2;
@@ -68,12 +66,12 @@ typedef struct TflGemm {
     const int32_t* slot;            /* cache row per batch row; negative: nothing is stored */
     int64_t ld_x, x_oct, x_group, ld_t, t_oct, ld_f, ld_gate, ld_tok, ld_kv;
     int32_t rows, n, k, groups;     /* n = outputs per group, all groups alike */
-    int32_t n_real, k_real, n_raw, ss_n, ss_ld;
+    int32_t n_real, k_real, n_raw, n_scaled, ss_n, ss_ld;
     int32_t H, N, R, C, half, c_real, max_pos, cache_rows, vocab;
     float eps;
 } TflGemm;
 
-int tfl_gemm(const TflGemm* a, int dtype, int x_mode, int epilogue, void* stream);
+int tfl_gemm(const TflGemm* a, int dtype, int epilogue, void* stream);
 
 /* x (fp32 residual) of one row per workgroup, in this order, each part optional:
  *   x = embed[ids]            (embed != NULL)

@@ -78,15 +78,17 @@ def test_input_projection(ol, dtype, rows, n_raw, n_up):
     k, off = 160, 64
     w, x = rnd(n_raw + n_up, k, seed=1, dtype=dtype, scale=k ** -0.5), rnd(rows, k, seed=2, dtype=dtype)
     act = torch.full((rows, off + n_up), 7.0, dtype=dtype, device=DEV)
-    raw, ss = ol.input_projection(x, ol.TileWeight(w), n_raw, act, off)
+    qw = rnd(96, seed=9)
+    raw, ss, xq = ol.input_projection(x, ol.TileWeight(w), n_raw, qw, act, off)
     want = f(x) @ f(w).T
     torch.testing.assert_close(raw, want[:, :n_raw], atol=1e-4, rtol=1e-4)
+    torch.testing.assert_close(f(ol.act_rows(xq)), want[:, :96] * qw, **OP[dtype])
     torch.testing.assert_close(ss, want[:, :n_raw].view(rows, -1, 16).pow(2).sum(-1), atol=1e-3, rtol=1e-3)
     torch.testing.assert_close(f(act[:, off:]), R.gelu(want[:, n_raw:]), **OP[dtype])
     assert bool((act[:, :off] == 7).all())
     block = torch.full(((off + n_up) // 8, rows, 8), 7.0, dtype=dtype, device=DEV)
-    raw2, ss2 = ol.input_projection(octets(x), ol.TileWeight(w), n_raw, block, off)
-    assert torch.equal(ol.act_rows(block), act) and torch.equal(raw2, raw) and torch.equal(ss2, ss)
+    raw2, ss2, xq2 = ol.input_projection(octets(x), ol.TileWeight(w), n_raw, qw, block, off)
+    assert torch.equal(ol.act_rows(block), act) and torch.equal(xq2, xq) and torch.equal(raw2, raw) and torch.equal(ss2, ss)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -107,9 +109,10 @@ def test_query_and_append(ol, dtype, rows, g):
     if rows > 2:
         slot[1] = -1                                              # an idle row stores nothing
     cache = torch.full((128, g.C + g.R), 5.0, dtype=dtype, device=DEV)
-    qn, q = ol.query_and_append(raw, ss, ol.TileWeight(w), g, qn_w, kv_w, eps, rope, pos, slot, cache)
-    cq = raw[:, :g.Q] / torch.sqrt(raw[:, :g.Q].pow(2).sum(-1, keepdim=True) / g.q_real + eps) * qn_w
-    full = (f(cq.to(dtype)) @ f(w).T).view(rows, g.H, g.N + g.R)
+    xq = octets((raw[:, :g.Q] * qn_w).to(dtype))
+    qn, q = ol.query_and_append(xq, raw, ss, ol.TileWeight(w), g, kv_w, eps, rope, pos, slot, cache)
+    cq = f(ol.act_rows(xq)) / torch.sqrt(raw[:, :g.Q].pow(2).sum(-1, keepdim=True) / g.q_real + eps)
+    full = (cq @ f(w).T).view(rows, g.H, g.N + g.R)
     torch.testing.assert_close(f(qn), full[..., :g.N], **OP[dtype])
     torch.testing.assert_close(f(q[..., g.C:]), rope.turn(full[..., g.N:], pos), **OP[dtype])
     c = raw[:, g.Q:g.Q + g.C]
@@ -149,13 +152,14 @@ def test_residual_and_token_gemms(ol, dtype, rows):
     w, a, x = rnd(96, 160, seed=1, dtype=dtype), rnd(rows, 160, seed=2, dtype=dtype), rnd(rows, 96, seed=3)
     want, x2 = x + f(a) @ f(w).T, x.clone()
     ol.add_linear(a, ol.TileWeight(w), x)
-    ol.add_linear(octets(a), ol.TileWeight(w), x2)
-    assert torch.equal(x, x2)
+    xt = ol.add_linear(octets(a), ol.TileWeight(w), x2, want_copy=True)
+    assert torch.equal(x, x2) and torch.equal(ol.act_rows(xt), x.to(dtype))
     torch.testing.assert_close(x, want, atol=1e-3, rtol=1e-4)
     w, table = rnd(32, 96, seed=4, dtype=dtype, scale=0.1), rnd(50, 60, seed=5, dtype=dtype)
     ids = torch.randint(0, 50, (rows,), generator=torch.Generator().manual_seed(1)).to(DEV)
     part = table[:, 20:43]
-    y = ol.token_gate_linear(x, ol.TileWeight(w), part, ids, 23)
+    y = ol.token_gate_linear(xt, ol.TileWeight(w), part, ids, 23)
+    assert torch.equal(ol.token_gate_linear(ol.act_rows(xt).contiguous(), ol.TileWeight(w), part, ids, 23), y)
     want = R.gelu((f(x.to(dtype)) @ f(w).T)[:, :23]) * f(part[ids])
     torch.testing.assert_close(f(y[:, :23]), want, **OP[dtype])
     assert bool((y[:, 23:] == 0).all())
@@ -291,7 +295,7 @@ def test_attn_decode_finds_one_key_anywhere(ol, dtype, heads, C, Rr):
             torch.testing.assert_close(out[b], f(keys[b][s, :C]).expand(heads, -1), atol=1e-2, rtol=1e-2)
 
 
-PRE_SHAPES = [(2, 32, 32, 32, 32), (3, 64, 32, 64, 96), (2, 128, 64, 128, 512), (2, 160, 64, 224, 320), (1, 320, 64, 256, 64)]
+PRE_SHAPES = [(2, 32, 32, 32, 32), (3, 64, 32, 64, 96), (2, 128, 64, 128, 512), (2, 160, 64, 224, 320), (1, 320, 64, 256, 64), (64, 128, 64, 128, 64)]
 
 
 def _prefill_case(g, news, pasts, dtype, seed):
@@ -323,11 +327,11 @@ def _prefill_want(g, q, kv, ck, seq, pos, rope, gate, scale):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("heads,N,Rr,V,C", PRE_SHAPES)
-@pytest.mark.parametrize("news,pasts", [((1,), (0,)), ((2, 1, 63, 65), (0, 0, 0, 0)), ((130, 5, 64), (0, 190, 64)), ((300,), (1,))])
+@pytest.mark.parametrize("news,pasts", [((1,), (0,)), ((2, 1, 63, 65), (0, 0, 0, 0)), ((130, 5, 64), (0, 190, 64)), ((300,), (1,)), ((520, 300), (0, 77))])
 def test_attn_prefill(ol, dtype, heads, N, Rr, V, C, news, pasts):
     g = Geom(heads, N, Rr, V, C, 32)
     q, kv, ck, seq, pos = _prefill_case(g, news, pasts, dtype, 3)
-    rope = Rope(400, Rr // 2)
+    rope = Rope(700, Rr // 2)
     tq = q.shape[0]
     gate = rnd(tq, g.H * g.V, seed=8, dtype=dtype)
     act = torch.full((tq, g.H * g.V + 32), 3.0, dtype=dtype, device=DEV)

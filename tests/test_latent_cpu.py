@@ -45,11 +45,11 @@ def test_bad_arguments_are_refused_before_any_launch():
     from triforce_amd import hip
     L = hip.latent_lib()
     a = hip.TflGemm()
-    assert L.tfl_gemm(ctypes.byref(a), 0, 0, 0, None) == -22
+    assert L.tfl_gemm(ctypes.byref(a), 0, 0, None) == -22
     a.wp = a.x = a.out_f = 1 << 20
     a.rows, a.n, a.k, a.groups, a.n_real, a.ld_f, a.ld_x = 1, 16, 32, 1, 16, 16, 32
     a.k = 40
-    assert L.tfl_gemm(ctypes.byref(a), 0, 0, 0, None) == -22
+    assert L.tfl_gemm(ctypes.byref(a), 0, 0, None) == -22
     assert L.tfl_attn_decode(1, 1, 1, 1, 1, 1, 1, None, 0, 1, 1, 48, 32, 1.0, 1, 0, None) == -22        # latent not padded
     assert L.tfl_attn_decode(1, 1, 1, 1, 1, 1, 1, None, 0, 1, 1, 64, 32, 1.0, 4, 0, None) == -28        # no workspace
     for rows in (1, 3, 64):

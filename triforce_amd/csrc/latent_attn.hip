@@ -2,13 +2,12 @@
 //
 // Decode (attn_latent_kernel): the query has been taken through the key up-projection, so the cached row itself is the key
 // ([latent | rotated]) and its latent part the value, for every head: one KV stream shared by all heads.  A workgroup walks the
-// 64-key pages of its split; the page goes global -> registers -> LDS (the next page's loads are in flight while this one is
-// used).  Scores are computed transposed (S^T = K Q^T: rows keys, columns heads), so that a lane owns one head's statistics;
+// 64-key pages of its split, staged in LDS.  Scores are computed transposed (S^T = K Q^T: rows keys, columns heads), so that a lane owns one head's statistics;
 // wave w takes keys 16w .. 16w+15.  The weights go to LDS as [head][key] and every wave then accumulates its share of the
 // latent columns, O^T = C^T P^T, with the transposed operand read straight from the key-major page (ds_read_b64_tr_b16).
 //
 // Prefill (attn_prefill_kernel): keys and values up-projected once per chunk, flash attention with 16 * QT query rows per wave,
-// four waves sharing the key / value tile.  Also transposed: the S^T result registers of two 16-key tiles ARE the P operand of
+// the waves of a workgroup sharing the key / value tile.  Also transposed: the S^T result registers of two 16-key tiles ARE the P operand of
 // one PV product (the value operand is read with the matching key order), so the weights never leave the registers.
 #include "latent_common.h"
 
@@ -46,9 +45,9 @@ __global__ __launch_bounds__(NW * 64, 1) void attn_latent_kernel(const T* __rest
 
     for (int p = tid; p < 16 * HT * ppr; p += NT) {           // queries of this head group (heads past H: zeros)
         const int r = p / ppr, c = p - r * ppr;
-        uint4 v = {0, 0, 0, 0};
-        if (h0 + r < H) v = *reinterpret_cast<const uint4*>(q + ((int64_t)row * H + h0 + r) * W + EPV * c);
-        *reinterpret_cast<uint4*>(Qs + r * ldk + EPV * c) = v;
+        u32x4 v = {0, 0, 0, 0};
+        if (h0 + r < H) v = *reinterpret_cast<const u32x4*>(q + ((int64_t)row * H + h0 + r) * W + EPV * c);
+        *reinterpret_cast<u32x4*>(Qs + r * ldk + EPV * c) = v;
     }
     auto page_base = [&](int t) {
         const int k0 = t * KT;
@@ -70,9 +69,9 @@ __global__ __launch_bounds__(NW * 64, 1) void attn_latent_kernel(const T* __rest
         const T* base = cache + page_base(t) * W;
         for (int p = tid; p < KT * ppr; p += NT) {
             const int r = p / ppr, c = p - r * ppr;
-            uint4 v = {0, 0, 0, 0};
-            if (k0 + r < n) v = *reinterpret_cast<const uint4*>(base + (int64_t)r * W + EPV * c);
-            *reinterpret_cast<uint4*>(Kt + r * ldk + EPV * c) = v;
+            u32x4 v = {0, 0, 0, 0};
+            if (k0 + r < n) v = *reinterpret_cast<const u32x4*>(base + (int64_t)r * W + EPV * c);
+            *reinterpret_cast<u32x4*>(Kt + r * ldk + EPV * c) = v;
         }
         __syncthreads();
         f32x4 s[HT];
@@ -277,7 +276,7 @@ __global__ __launch_bounds__(256 * HT, HT) void attn_latent_sized_kernel(const b
             if (head >= H) qf[c] = bf16x8{};
         }
     }
-    uint4 pre[NPRE];
+    u32x4 pre[NPRE];
     auto page_of = [&](int t) {
         const int pg = tab[t];
         return pg < 0 ? 0 : (pg >= n_pages ? n_pages - 1 : pg);
@@ -285,7 +284,7 @@ __global__ __launch_bounds__(256 * HT, HT) void attn_latent_sized_kernel(const b
     auto fetch = [&](int pg) {
         const bf16* base = cache + (int64_t)pg * (64 * W) + tid * 8;
 #pragma unroll
-        for (int j = 0; j < NPRE; ++j) pre[j] = *reinterpret_cast<const uint4*>(base + j * NT * 8);
+        for (int j = 0; j < NPRE; ++j) pre[j] = *reinterpret_cast<const u32x4*>(base + j * NT * 8);
     };
     auto put = [&](int t) {
         bf16* dst = Kt + (t & 1) * 64 * LDK;
@@ -293,9 +292,9 @@ __global__ __launch_bounds__(256 * HT, HT) void attn_latent_sized_kernel(const b
 #pragma unroll
         for (int j = 0; j < NPRE; ++j) {
             const int p = tid + j * NT, r = p / (W / 8), c = p - r * (W / 8);
-            uint4 v = pre[j];
-            if (edge && 64 * t + r >= n) v = uint4{0, 0, 0, 0};     // rows past the end: never let stale contents into 0 * x
-            *reinterpret_cast<uint4*>(dst + r * LDK + 8 * c) = v;
+            u32x4 v = pre[j];
+            if (edge && 64 * t + r >= n) v = u32x4{0, 0, 0, 0};     // rows past the end: never let stale contents into 0 * x
+            *reinterpret_cast<u32x4*>(dst + r * LDK + 8 * c) = v;
         }
     };
     f32x4 o[HT][NTW];
@@ -520,12 +519,26 @@ extern "C" int tfl_attn_decode(const void* q, const void* cache, int n_pages, co
 }
 
 // --------------------------------------------------------------------------------------------------------------- prefill
-template <int V> struct Int { static constexpr int value = V; };
+// A 64-row section of PR 16-byte pieces per row, spread over NT threads, to / from registers pre[AT ..].
+template <int NT, int PR, int AT, typename T, int N>
+__device__ __forceinline__ void fetch_section(u32x4 (&pre)[N], const T* base, int64_t ld, int left, int tid) {
+    const int r0 = tid / PR, c = tid % PR;
+#pragma unroll
+    for (int j = 0; j < 64 * PR / NT; ++j)
+        if (AT + j < N) pre[AT + j] = *reinterpret_cast<const u32x4*>(base + (int64_t)min(r0 + j * (NT / PR), left) * ld + 8 * c);
+}
+template <int NT, int PR, int AT, typename T, int N>
+__device__ __forceinline__ void put_section(const u32x4 (&pre)[N], T* base, int ld, int tid) {
+    const int r0 = tid / PR, c = tid % PR;
+#pragma unroll
+    for (int j = 0; j < 64 * PR / NT; ++j)
+        if (AT + j < N) *reinterpret_cast<u32x4*>(base + (r0 + j * (NT / PR)) * ld + 8 * c) = pre[AT + j];
+}
 
-// KT keys per tile, QT 16-row query tiles per wave, up to DK 32-wide chunks of query-key size (NC unrotated ones first) and DV
+// NWV waves, KT keys per tile, QT 16-row query tiles per wave, up to DK 32-wide chunks of query-key size (NC unrotated ones first) and DV
 // 16-wide tiles of value size.  EXACT: the sizes are exactly NCX, DK, DV (no bounds in the inner loops, register look-ahead).
-template <typename T, int KT, int QT, int DK, int DV, int NCX>
-__global__ __launch_bounds__(256, NCX > 0 ? 2 : 1) void attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ kv, const T* __restrict__ ck,
+template <typename T, int NWV, int KT, int QT, int DK, int DV, int NCX>
+__global__ __launch_bounds__(64 * NWV, NWV / 4) void attn_prefill_kernel(const T* __restrict__ q, const T* __restrict__ kv, const T* __restrict__ ck,
                                                            const int32_t* __restrict__ seq, const int32_t* __restrict__ pos,
                                                            const float* __restrict__ cosb, const float* __restrict__ sinb,
                                                            int half, int max_pos, const T* __restrict__ gate, int64_t ld_gate,
@@ -533,12 +546,12 @@ __global__ __launch_bounds__(256, NCX > 0 ? 2 : 1) void attn_prefill_kernel(cons
                                                            int V, int C, float scale) {
     typedef typename El<T>::Frag Frag;
     constexpr bool EXACT = NCX > 0;
-    constexpr int EPV = 16 / sizeof(T), PADE = EPV, QB = 64 * QT;
+    constexpr int EPV = 16 / sizeof(T), PADE = EPV, PADV = 2 * EPV, QB = 16 * NWV * QT, NT = 64 * NWV;
     extern __shared__ __align__(16) char smem[];
     const int nc = EXACT ? NCX : N >> 5, dk = EXACT ? DK : (N + R) >> 5, dv = EXACT ? DV : V >> 4;
-    const int D = 32 * dk, ldk = D + PADE, ldv = 16 * dv + PADE;
-    T* Ks = (T*)smem;                                         // [KT][ldk]
-    T* Vs = Ks + KT * ldk;                                    // [KT][ldv]
+    const int D = 32 * dk, ldk = D + PADE, ldv = 16 * dv + PADV;
+    T* Ks = (T*)smem;                                         // [1 or 2][KT][ldk], then the values [KT][ldv]
+    T* Vs = Ks + (EXACT ? 2 : 1) * KT * ldk;
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g = lane >> 4, i = lane & 15;
     // workgroups go round-robin over the 8 XCDs: all query blocks of a head sit on one of them and share its L2, longest first
     const int nqb = gridDim.x / H, id = blockIdx.x;
@@ -592,42 +605,38 @@ __global__ __launch_bounds__(256, NCX > 0 ? 2 : 1) void attn_prefill_kernel(cons
     const int ntiles = (past + last_q) / KT + 1;
     const int first_qpos = past + qb + 16 * wave * QT;        // the wave's first row: tiles that end before it need no mask
     [[maybe_unused]] const int kn = N / EPV, kr = R / EPV, vn = V / EPV, ppr = kn + kr + vn;   // 16-byte pieces per key
-    // EXACT: a tile is NJ pieces per thread; piece j of a section is row (tid / pieces per row) + j * step of it
-    constexpr int RCX = EXACT ? DK - NCX : 1, NKX = EXACT ? NCX : 1, JV = EXACT ? DV / 2 : 1, NJ = EXACT ? NKX + RCX + JV : 1;
-    static_assert(!EXACT || (KT == 64 && 256 % (4 * NKX) == 0 && 256 % (4 * RCX) == 0 && 256 % (4 * JV) == 0), "piece split");
-    uint4 pre[NJ];
+    // EXACT: two tiles in LDS and one in registers.  A tile is NJ pieces per thread; piece j of a section is row
+    // (tid / pieces per row) + j * step of it
+    constexpr int RCX = EXACT ? DK - NCX : 1, NKX = EXACT ? NCX : 1, VCX = EXACT ? DV / 2 : 1;
+    constexpr int NJ = EXACT ? 4 * (NKX + RCX + VCX) / NWV : 1;
+    static_assert(!EXACT || (KT == 64 && (4 * NKX) % NWV == 0 && (4 * RCX) % NWV == 0 && (4 * VCX) % NWV == 0), "piece split");
+    u32x4 pre[NJ];
     auto fetch = [&](int t) {
         const T* kv_t = kv + (int64_t)(k_at + t * KT) * ld_kv;
         const T* ck_t = ck + (int64_t)(k_at + t * KT) * ld_ck + C;
         const int left = nk - t * KT - 1;                     // rows past the last key repeat it (masked)
-        auto section = [&](auto per_row, auto count, int at, const T* base, int64_t ld) {
-            const int r0 = tid / per_row.value, c = tid % per_row.value;
-#pragma unroll
-            for (int j = 0; j < count.value; ++j)
-                pre[at + j] = *reinterpret_cast<const uint4*>(base + (int64_t)min(r0 + j * (256 / per_row.value), left) * ld + 8 * c);
-        };
-        section(Int<4 * NKX>{}, Int<NKX>{}, 0, kv_t + (int64_t)h * N, ld_kv);
-        section(Int<4 * RCX>{}, Int<RCX>{}, NKX, ck_t, ld_ck);
-        section(Int<4 * JV>{}, Int<JV>{}, NKX + RCX, kv_t + (int64_t)H * N + (int64_t)h * V, ld_kv);
+        fetch_section<NT, 4 * NKX, 0>(pre, kv_t + (int64_t)h * N, ld_kv, left, tid);
+        fetch_section<NT, 4 * RCX, 4 * NKX / NWV>(pre, ck_t, ld_ck, left, tid);
+        fetch_section<NT, 4 * VCX, 4 * (NKX + RCX) / NWV>(pre, kv_t + (int64_t)H * N + (int64_t)h * V, ld_kv, left, tid);
     };
-    auto put = [&]() {
-        auto section = [&](auto per_row, auto count, int at, T* base, int ld) {
-            const int r0 = tid / per_row.value, c = tid % per_row.value;
-#pragma unroll
-            for (int j = 0; j < count.value; ++j)
-                *reinterpret_cast<uint4*>(base + (r0 + j * (256 / per_row.value)) * ld + 8 * c) = pre[at + j];
-        };
-        section(Int<4 * NKX>{}, Int<NKX>{}, 0, Ks, ldk);
-        section(Int<4 * RCX>{}, Int<RCX>{}, NKX, Ks + 32 * NKX, ldk);
-        section(Int<4 * JV>{}, Int<JV>{}, NKX + RCX, Vs, ldv);
+    auto put = [&](int t) {
+        T* kt = Ks + (t & 1) * KT * ldk;
+        put_section<NT, 4 * NKX, 0>(pre, kt, ldk, tid);
+        put_section<NT, 4 * RCX, 4 * NKX / NWV>(pre, kt + 32 * NKX, ldk, tid);
+        put_section<NT, 4 * VCX, 4 * (NKX + RCX) / NWV>(pre, Vs + (t & 1) * KT * ldv, ldv, tid);
     };
-    if constexpr (EXACT) fetch(0);
+    if constexpr (EXACT) {
+        fetch(0);
+        put(0);
+        if (ntiles > 1) fetch(1);
+        __syncthreads();
+    }
     for (int t = 0; t < ntiles; ++t) {
         const int k0 = t * KT;
-        if constexpr (EXACT) {
-            put();
-        } else {
-            for (int p = tid; p < KT * ppr; p += 256) {
+        const T* Kt = EXACT ? Ks + (t & 1) * KT * ldk : Ks;
+        const T* Vt = EXACT ? Vs + (t & 1) * KT * ldv : Vs;
+        if constexpr (!EXACT) {
+            for (int p = tid; p < KT * ppr; p += NT) {
                 const int key = p / ppr;
                 int c = p - key * ppr;
                 const int64_t kk = k_at + min(k0 + key, nk - 1);
@@ -645,16 +654,16 @@ __global__ __launch_bounds__(256, NCX > 0 ? 2 : 1) void attn_prefill_kernel(cons
                     src = kv + kk * ld_kv + (int64_t)H * N + (int64_t)h * V + EPV * c;
                     dst = Vs + key * ldv + EPV * c;
                 }
-                *reinterpret_cast<uint4*>(dst) = *reinterpret_cast<const uint4*>(src);
+                *reinterpret_cast<u32x4*>(dst) = *reinterpret_cast<const u32x4*>(src);
             }
+            __syncthreads();
         }
-        __syncthreads();
         f32x4 s[KT / 16][QT];
 #pragma unroll
         for (int kt = 0; kt < KT / 16; ++kt) {
 #pragma unroll
             for (int u = 0; u < QT; ++u) s[kt][u] = f32x4{0.f, 0.f, 0.f, 0.f};
-            const T* kp = Ks + (16 * kt + i) * ldk + 8 * g;
+            const T* kp = Kt + (16 * kt + i) * ldk + 8 * g;
 #pragma unroll
             for (int c = 0; c < DK; ++c) {
                 if (EXACT || c < dk) {
@@ -703,15 +712,16 @@ __global__ __launch_bounds__(256, NCX > 0 ? 2 : 1) void attn_prefill_kernel(cons
                     for (int r = 0; r < 4; ++r) o[u][d][r] *= alpha;
             }
         }
-        if constexpr (EXACT) {                                // (here the score registers are free: two workgroups fit a CU)
-            if (t + 1 < ntiles) fetch(t + 1);
+        if constexpr (EXACT) {
+            if (t + 1 < ntiles) put(t + 1);
+            if (t + 2 < ntiles) fetch(t + 2);
         }
 #pragma unroll
         for (int d = 0; d < DV; ++d) {
             if (EXACT || d < dv) {
 #pragma unroll
                 for (int c = 0; c < KT / 32; ++c) {
-                    const Frag a = load_frag_t(Vs, ldv, 32 * c + 4 * g, 32 * c + 16 + 4 * g, 16 * d, i);
+                    const Frag a = load_frag_t(Vt, ldv, 32 * c + 4 * g, 32 * c + 16 + 4 * g, 16 * d, i);
 #pragma unroll
                     for (int u = 0; u < QT; ++u) o[u][d] = El<T>::mma(a, pf[u][c], o[u][d]);
                 }
@@ -741,21 +751,21 @@ __global__ __launch_bounds__(256, NCX > 0 ? 2 : 1) void attn_prefill_kernel(cons
     }
 }
 
-template <typename T, int KT, int QT, int DK, int DV, int NCX>
+template <typename T, int NWV, int KT, int QT, int DK, int DV, int NCX>
 static int launch_prefill(const void* q, const void* kv, const void* ck, const int32_t* seq, int nseq, int max_new, const int32_t* pos,
                           const float* cosb, const float* sinb, int half, int max_pos, const void* gate, int64_t ld_gate, void* out,
                           int64_t ld_out, int tq, int tk, int H, int N, int R, int V, int C, float scale, hipStream_t st) {
     const int pad = 16 / (int)sizeof(T);
-    const size_t lds = sizeof(T) * KT * (size_t)(N + R + V + 2 * pad);
+    const size_t lds = (NCX > 0 ? 2 : 1) * sizeof(T) * KT * (size_t)(N + R + V + 3 * pad);
     if (lds > 160 * 1024) return TF_ERANGE;
-    auto k = attn_prefill_kernel<T, KT, QT, DK, DV, NCX>;
+    auto k = attn_prefill_kernel<T, NWV, KT, QT, DK, DV, NCX>;
     static bool attr = false;
     if (!attr) {
         const hipError_t e = hipFuncSetAttribute((const void*)k, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
         if (e != hipSuccess) return (int)e;
         attr = true;
     }
-    hipLaunchKernelGGL(k, dim3((max_new + 64 * QT - 1) / (64 * QT) * H, nseq), dim3(256), lds, st, (const T*)q, (const T*)kv, (const T*)ck,
+    hipLaunchKernelGGL(k, dim3((max_new + 16 * NWV * QT - 1) / (16 * NWV * QT) * H, nseq), dim3(64 * NWV), lds, st, (const T*)q, (const T*)kv, (const T*)ck,
                        seq, pos, cosb, sinb, half, max_pos, (const T*)gate, ld_gate, (T*)out, ld_out, tq, tk, H, N, R, V, C, scale);
     TFL_LAUNCH_CHECK();
     return TF_OK;
@@ -770,21 +780,24 @@ extern "C" int tfl_attn_prefill(const void* q, const void* kv, const void* ck, c
     if (half < 0 || 2 * half > R || max_pos < 1 || (half && (!cosb || !sinb)) || !(scale > 0.f)) return TF_EINVAL;
     if ((ld_gate & 3) || (ld_out & 3) || ld_gate < (int64_t)H * V || ld_out < (int64_t)H * V) return TF_EINVAL;
     hipStream_t st = (hipStream_t)stream;
-#define GO(T, KT, QT, DK, DV, NCX)                                                                                               \
-    return launch_prefill<T, KT, QT, DK, DV, NCX>(q, kv, ck, seq, nseq, max_new, pos, cosb, sinb, half, max_pos, gate, ld_gate, \
+#define GO(T, NWV, KT, QT, DK, DV, NCX)                                                                                               \
+    return launch_prefill<T, NWV, KT, QT, DK, DV, NCX>(q, kv, ck, seq, nseq, max_new, pos, cosb, sinb, half, max_pos, gate, ld_gate, \
                                                   out, ld_out, tq, tk, H, N, R, V, C, scale, st)
     const int D = N + R;
     if (dtype == 0) {
-        if (N == 128 && R == 64 && V == 128) GO(bf16, 64, 2, 6, 8, 4);
-        if (D <= 96 && V <= 64) GO(bf16, 64, 1, 3, 4, 0);
-        if (D <= 192 && V <= 128) GO(bf16, 64, 1, 6, 8, 0);
-        if (D <= 384 && V <= 256) GO(bf16, 64, 1, 12, 16, 0);
+        if (N == 128 && R == 64 && V == 128) {                   // 256 query rows per workgroup where that still fills the chip
+            if ((int64_t)((max_new + 255) / 256) * H * nseq >= 256) GO(bf16, 8, 64, 2, 6, 8, 4);
+            GO(bf16, 4, 64, 2, 6, 8, 4);
+        }
+        if (D <= 96 && V <= 64) GO(bf16, 4, 64, 1, 3, 4, 0);
+        if (D <= 192 && V <= 128) GO(bf16, 4, 64, 1, 6, 8, 0);
+        if (D <= 384 && V <= 256) GO(bf16, 4, 64, 1, 12, 16, 0);
         return TF_ERANGE;
     }
     if (dtype == 1) {
-        if (D <= 96 && V <= 64) GO(float, 32, 1, 3, 4, 0);
-        if (D <= 192 && V <= 128) GO(float, 32, 1, 6, 8, 0);
-        if (D <= 384 && V <= 256) GO(float, 32, 1, 12, 16, 0);
+        if (D <= 96 && V <= 64) GO(float, 4, 32, 1, 3, 4, 0);
+        if (D <= 192 && V <= 128) GO(float, 4, 32, 1, 6, 8, 0);
+        if (D <= 384 && V <= 256) GO(float, 4, 32, 1, 12, 16, 0);
         return TF_ERANGE;
     }
 #undef GO

@@ -3,12 +3,14 @@
 // csrc/gemv.hip (a wave's weight load is one contiguous run per 16x32 tile, partial tiles meet in LDS), with the element type
 // a template parameter and the epilogues of this family:
 //   IN        the four projections that read the layer's one norm (query latent, key latent | key, gate, feed-forward up):
-//             raw fp32 outputs plus per-panel sums of squares (the norms of the two latents need them), gelu on the last part
-//   QUERY     query latent normalised in the operand load, heads written as unrotated | rotated; spare workgroups of the same
-//             launch normalise, rotate and store the cache rows
+//             raw fp32 outputs plus per-panel sums of squares, the query latent also times its norm weight as the next operand
+//             (its row scale is applied behind the next product), gelu on the last part
+//   QUERY     row scale from the sums of squares, heads written as unrotated | rotated; spare workgroups of the same launch
+//             normalise, rotate and store the cache rows
 //   LATENT    per head: query through the transposed key up-projection, next to the rotated part
 //   GATED     per head: value up-projection of the attended latent, times the output gate
 //   RESIDUAL  attention output and feed-forward down in one matrix, added to the fp32 residual
+//             (and the sum again as the next operand)
 //   TOKEN     per-layer token input: gelu times the token's row of a table
 #include "latent_common.h"
 
@@ -16,15 +18,11 @@
 #define TFL_PAIR_MIN 420     // panel pairs from which two panels share a workgroup
 #endif
 
-template <typename T, int XMODE> struct RawX { typedef f32x8 Type; };
-template <typename T> struct RawX<T, TFL_X_T> { typedef typename El<T>::Frag Type; };
-
 // P panels per workgroup (they share the operand rows), MT 16-row blocks, U tiles of 32 per batch; AHEAD: the next batch's weights
 // are requested before the current one is used (long K), otherwise a wave's whole K range should fit one or two batches.
-template <typename T, int XMODE, int EPI, int P, int MT, int WAVES, int U, bool AHEAD>
+template <typename T, int EPI, int P, int MT, int WAVES, int U, bool AHEAD>
 __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a) {
     typedef typename El<T>::Frag Frag;
-    typedef typename RawX<T, XMODE>::Type Raw;
     static_assert(P * MT <= WAVES, "one wave finishes one 16x16 tile");
     __shared__ f32x4 part[WAVES][P * MT][64];
     const int ppg = a.n >> 4, npan = ppg * a.groups;
@@ -44,7 +42,7 @@ __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a
             return;
         }
     }
-    const int wave = tid >> 6, lane = tid & 63, g = lane >> 4, i = lane & 15;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, g = lane >> 4, i = lane & 15;
     const int panel0 = blockIdx.x * P, grp = P == 1 ? panel0 / ppg : 0;
     const int m0 = blockIdx.y * 16 * MT;
     const int chunks = a.k >> 5;
@@ -54,18 +52,17 @@ __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a
 #pragma unroll
     for (int p = 0; p < P; ++p) wp[p] = (const T*)a.wp + (int64_t)min(panel0 + p, npan - 1) * chunks * 512 + lane * 8;
     int64_t xoff[MT];
-    int mrow[MT];
 #pragma unroll
-    for (int t = 0; t < MT; ++t) {
-        mrow[t] = min(m0 + 16 * t + i, a.rows - 1);
-        xoff[t] = (int64_t)mrow[t] * a.ld_x + (int64_t)grp * a.x_group + g * a.x_oct;
-    }
+    for (int t = 0; t < MT; ++t)
+        xoff[t] = (int64_t)min(m0 + 16 * t + i, a.rows - 1) * a.ld_x + (int64_t)grp * a.x_group + g * a.x_oct;
     const int64_t xstep = 4 * a.x_oct;
     auto load_w = [&](Frag (&w)[P][U], int c0) {
 #pragma unroll
         for (int u = 0; u < U; ++u)
+            if (AHEAD || c0 + u < c_end) {                    // (AHEAD: straight-line code, the tail repeats the last tile)
 #pragma unroll
-            for (int p = 0; p < P; ++p) w[p][u] = load_frag_stream(wp[p] + (int64_t)min(c0 + u, last) * 512);
+                for (int p = 0; p < P; ++p) w[p][u] = load_frag_stream(wp[p] + (int64_t)min(c0 + u, last) * 512);
+            }
     };
     f32x4 acc[P][MT];
 #pragma unroll
@@ -73,55 +70,24 @@ __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a
 #pragma unroll
         for (int t = 0; t < MT; ++t) acc[p][t] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (c_beg < c_end) {
-        float inv[MT];
-        bool scaled = false;
         Frag w[P][U], wn[P][U];
         load_w(w, c_beg);
         for (int c0 = c_beg; c0 < c_end; c0 += U) {
-            Raw xr[U][MT];
-            f32x8 nw[U];
+            Frag x[U][MT];
 #pragma unroll
-            for (int u = 0; u < U; ++u) {
-                const int c = min(c0 + u, last);
+            for (int u = 0; u < U; ++u)
+                if (AHEAD || c0 + u < c_end) {
 #pragma unroll
-                for (int t = 0; t < MT; ++t) {
-                    if constexpr (XMODE == TFL_X_T) xr[u][t] = load_frag((const T*)a.x + xoff[t] + xstep * c);
-                    else xr[u][t] = *reinterpret_cast<const f32x8*>((const float*)a.x + xoff[t] + xstep * c);
+                    for (int t = 0; t < MT; ++t) x[u][t] = load_frag((const T*)a.x + xoff[t] + xstep * min(c0 + u, last));
                 }
-                if constexpr (XMODE == TFL_X_F32_NORM) nw[u] = *reinterpret_cast<const f32x8*>((const float*)a.norm_w + 32 * c + 8 * g);
-            }
             if constexpr (AHEAD) load_w(wn, c0 + U);
-            if constexpr (XMODE == TFL_X_F32_NORM) {         // the row's scale from the producer's per-panel sums of squares
-                if (!scaled) {
-#pragma unroll
-                    for (int t = 0; t < MT; ++t) {
-                        float s = 0.f;
-#pragma unroll 4
-                        for (int p = g; p < a.ss_n; p += 4) s += a.ss_in[(int64_t)mrow[t] * a.ss_ld + p];
-                        s += __shfl_xor(s, 16, 64);
-                        s += __shfl_xor(s, 32, 64);
-                        inv[t] = 1.0f / sqrtf(s / (float)a.k_real + a.eps);
-                    }
-                    scaled = true;
-                }
-            }
 #pragma unroll
             for (int u = 0; u < U; ++u)
                 if (c0 + u < c_end) {
 #pragma unroll
-                    for (int t = 0; t < MT; ++t) {
-                        Frag x;
-                        if constexpr (XMODE == TFL_X_T) x = xr[u][t];
-                        else {
+                    for (int t = 0; t < MT; ++t)
 #pragma unroll
-                            for (int e = 0; e < 8; ++e) {
-                                if constexpr (XMODE == TFL_X_F32_NORM) x[e] = (T)(xr[u][t][e] * inv[t] * nw[u][e]);
-                                else x[e] = (T)xr[u][t][e];
-                            }
-                        }
-#pragma unroll
-                        for (int p = 0; p < P; ++p) acc[p][t] = El<T>::mma(w[p][u], x, acc[p][t]);
-                    }
+                        for (int p = 0; p < P; ++p) acc[p][t] = El<T>::mma(w[p][u], x[u][t], acc[p][t]);
                 }
             if constexpr (AHEAD) {
 #pragma unroll
@@ -137,6 +103,21 @@ __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a
     for (int p = 0; p < P; ++p)
 #pragma unroll
         for (int t = 0; t < MT; ++t) part[wave][p * MT + t][lane] = acc[p][t];
+    float inv = 1.f;
+    if constexpr (EPI == TFL_EPI_QUERY) {                    // scale of row m from the producer's per-panel sums of squares
+        if (wave < MT) {
+            const float2* ss = reinterpret_cast<const float2*>(a.ss_in + (int64_t)min(m0 + 16 * wave + i, a.rows - 1) * a.ss_ld);
+            float q = 0.f;
+#pragma unroll 8
+            for (int p = g; p < a.ss_n / 2; p += 4) {
+                const float2 v = ss[p];
+                q += v.x + v.y;
+            }
+            q += __shfl_xor(q, 16, 64);
+            q += __shfl_xor(q, 32, 64);
+            inv = 1.0f / sqrtf(q / (float)a.k_real + a.eps);
+        }
+    }
     __syncthreads();
     if (wave >= P * MT) return;                              // wave p * MT + t finishes row block t of panel p
     const int t = wave % MT, panel = panel0 + wave / MT, pin = P == 1 ? panel - grp * ppg : panel;
@@ -158,6 +139,12 @@ __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a
             q += __shfl_xor(q, 32, 64);
             if (live) {
                 *reinterpret_cast<f32x4*>(a.out_f + (int64_t)m * a.ld_f + n) = s;
+                if (n < a.n_scaled) {
+                    const f32x4 w = *reinterpret_cast<const f32x4*>(a.norm_w + n);
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) s[r] *= w[r];
+                    store_quad((T*)a.out_t2 + (int64_t)m * 8 + (n >> 3) * (8 * (int64_t)a.rows) + (n & 7), s);
+                }
                 if (g == 0) a.ss_out[(int64_t)m * a.ss_ld + pin] = q;
             }
         } else if (live) {
@@ -175,6 +162,8 @@ __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a
         for (int r = 0; r < 4; ++r)
             if (n + r < a.n_real) y[r] = s[r];
     } else if constexpr (EPI == TFL_EPI_QUERY) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s[r] *= inv;
         const int per_head = a.N + a.R, h = n / per_head, e = n - h * per_head;
         const int64_t row = (int64_t)m * a.H + h;
         if (e < a.N) {
@@ -209,6 +198,7 @@ __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a
 #pragma unroll
         for (int r = 0; r < 4; ++r) o[r] += s[r];
         *y = o;
+        if (a.out_t) store_quad((T*)a.out_t + (int64_t)m * a.ld_t + (n >> 3) * a.t_oct + (n & 7), o);
     } else if constexpr (EPI == TFL_EPI_TOKEN) {
         int64_t id = a.ids[m];
         id = id < 0 ? 0 : (id >= a.vocab ? a.vocab - 1 : id);
@@ -219,56 +209,52 @@ __global__ __launch_bounds__(WAVES * 64) void latent_gemm_kernel(const TflGemm a
     }
 }
 
-template <typename T, int XMODE, int EPI, int P, int WAVES, int U, bool AHEAD>
+template <typename T, int EPI, int P, int WAVES, int U, bool AHEAD>
 static int launch_form(const TflGemm& a, hipStream_t st) {
     const int panels = (a.n >> 4) * a.groups;
     const int mt = a.rows <= 16 ? 1 : 2, rb = (a.rows + 16 * mt - 1) / (16 * mt);
     const int extra = EPI == TFL_EPI_QUERY && a.kv_raw ? (a.rows + rb - 1) / rb : 0;
     const dim3 grid((panels + P - 1) / P + extra, rb), block(64 * WAVES);
-    if (mt == 1) hipLaunchKernelGGL((latent_gemm_kernel<T, XMODE, EPI, P, 1, WAVES, U, AHEAD>), grid, block, 0, st, a);
-    else hipLaunchKernelGGL((latent_gemm_kernel<T, XMODE, EPI, P, 2, WAVES, U, AHEAD>), grid, block, 0, st, a);
+    if (mt == 1) hipLaunchKernelGGL((latent_gemm_kernel<T, EPI, P, 1, WAVES, U, AHEAD>), grid, block, 0, st, a);
+    else hipLaunchKernelGGL((latent_gemm_kernel<T, EPI, P, 2, WAVES, U, AHEAD>), grid, block, 0, st, a);
     TFL_LAUNCH_CHECK();
     return TF_OK;
 }
 
-// Waves per panel by panel count (few panels: more waves keep the weight stream deep enough); wide outputs take two panels per
-// workgroup.  The small per-head / latent products issue a wave's whole K range at once.
-template <typename T, int XMODE, int EPI>
+// Waves per panel by panel count (few panels: more waves keep the weight stream deep enough); wide outputs of more than 16 rows
+// take two panels per workgroup.  The small products issue a wave's whole K range at once.
+template <typename T, int EPI>
 static int launch_gemm(const TflGemm& a, hipStream_t st) {
     const int panels = (a.n >> 4) * a.groups;
     if constexpr (sizeof(T) == 4) {
-        return launch_form<T, XMODE, EPI, 1, 8, 2, true>(a, st);
+        return launch_form<T, EPI, 1, 8, 2, true>(a, st);
     } else if constexpr (EPI == TFL_EPI_IN || EPI == TFL_EPI_F32 || EPI == TFL_EPI_RESIDUAL) {
-        if (panels >= 2 * TFL_PAIR_MIN) return launch_form<T, XMODE, EPI, 2, 4, 4, true>(a, st);
-        if (panels > 512) return launch_form<T, XMODE, EPI, 1, 4, 4, true>(a, st);
-        if (panels > 128) return launch_form<T, XMODE, EPI, 1, 8, 4, true>(a, st);
-        return launch_form<T, XMODE, EPI, 1, 16, 4, true>(a, st);
-    } else if constexpr (XMODE != TFL_X_T) {                  // (fp32 operands: registers for half the batch)
-        if (panels > 512) return launch_form<T, XMODE, EPI, 1, 4, 4, true>(a, st);
-        if (panels > 128 || EPI == TFL_EPI_QUERY) return launch_form<T, XMODE, EPI, 1, 8, 4, true>(a, st);
-        return launch_form<T, XMODE, EPI, 1, 16, 4, true>(a, st);
+        if (panels >= 2 * TFL_PAIR_MIN && a.rows > 16) return launch_form<T, EPI, 2, 4, 4, true>(a, st);
+        if (panels > 512) return launch_form<T, EPI, 1, 4, 4, true>(a, st);
+        if (panels > 128) return launch_form<T, EPI, 1, 8, 4, true>(a, st);
+        return launch_form<T, EPI, 1, 16, 4, true>(a, st);
     } else {
-        if (panels > 512) return launch_form<T, XMODE, EPI, 1, 4, 8, false>(a, st);
-        if (panels > 128) return launch_form<T, XMODE, EPI, 1, 8, 8, false>(a, st);
-        return launch_form<T, XMODE, EPI, 1, 16, 8, false>(a, st);
+        if (panels > 512) return launch_form<T, EPI, 1, 4, 8, false>(a, st);
+        if (panels > 128) return launch_form<T, EPI, 1, 8, 8, false>(a, st);
+        return launch_form<T, EPI, 1, 16, 8, false>(a, st);
     }
 }
 
 template <typename T>
-static int dispatch_gemm(const TflGemm& a, int x_mode, int epi, hipStream_t st) {
-#define CASE(X, E) if (x_mode == X && epi == E) return launch_gemm<T, X, E>(a, st);
-    CASE(TFL_X_T, TFL_EPI_F32)
-    CASE(TFL_X_T, TFL_EPI_IN)
-    CASE(TFL_X_F32_NORM, TFL_EPI_QUERY)
-    CASE(TFL_X_T, TFL_EPI_LATENT)
-    CASE(TFL_X_T, TFL_EPI_GATED)
-    CASE(TFL_X_T, TFL_EPI_RESIDUAL)
-    CASE(TFL_X_F32, TFL_EPI_TOKEN)
-#undef CASE
+static int dispatch_gemm(const TflGemm& a, int epi, hipStream_t st) {
+    switch (epi) {
+        case TFL_EPI_F32: return launch_gemm<T, TFL_EPI_F32>(a, st);
+        case TFL_EPI_IN: return launch_gemm<T, TFL_EPI_IN>(a, st);
+        case TFL_EPI_QUERY: return launch_gemm<T, TFL_EPI_QUERY>(a, st);
+        case TFL_EPI_LATENT: return launch_gemm<T, TFL_EPI_LATENT>(a, st);
+        case TFL_EPI_GATED: return launch_gemm<T, TFL_EPI_GATED>(a, st);
+        case TFL_EPI_RESIDUAL: return launch_gemm<T, TFL_EPI_RESIDUAL>(a, st);
+        case TFL_EPI_TOKEN: return launch_gemm<T, TFL_EPI_TOKEN>(a, st);
+    }
     return TF_EINVAL;
 }
 
-extern "C" int tfl_gemm(const TflGemm* p, int dtype, int x_mode, int epi, void* stream) {
+extern "C" int tfl_gemm(const TflGemm* p, int dtype, int epi, void* stream) {
     if (!p || !p->wp || !p->x) return TF_EINVAL;
     const TflGemm a = *p;
     if (a.rows < 1 || a.rows > (1 << 20) || a.n < 16 || (a.n & 15) || a.k < 32 || (a.k & 31) || a.groups < 1) return TF_EINVAL;
@@ -281,13 +267,14 @@ extern "C" int tfl_gemm(const TflGemm* p, int dtype, int x_mode, int epi, void* 
             break;
         case TFL_EPI_IN:
             if (!a.out_f || !a.ss_out || a.groups != 1 || a.n_raw < 16 || (a.n_raw & 15) || a.n_raw > a.n || a.ld_f < a.n_raw
-                || (a.ld_f & 3) || a.ss_ld < a.n_raw / 16) return TF_EINVAL;
+                || (a.ld_f & 3) || a.ss_ld < a.n_raw / 16 || a.n_scaled < 0
+                || (a.n_scaled & 15) || a.n_scaled > a.n_raw || (a.n_scaled && (!a.norm_w || !a.out_t2))) return TF_EINVAL;
             if (a.n_raw < a.n && (!a.out_t || (a.ld_t & 7) || a.ld_t < 8)) return TF_EINVAL;
             break;
         case TFL_EPI_QUERY:
             if (!a.out_t || !a.out_t2 || !a.pos || a.groups != 1 || a.H < 1 || a.N < 16 || a.R < 0 || a.C < 16) return TF_EINVAL;
             if ((a.N & 15) || (a.R & 15) || (a.C & 15) || a.n != a.H * (a.N + a.R)) return TF_EINVAL;
-            if (!a.norm_w || !a.ss_in || a.ss_n < 1 || a.ss_ld < a.ss_n || a.k_real < 1 || a.k_real > a.k) return TF_EINVAL;
+            if (!a.ss_in || a.ss_n < 2 || (a.ss_n & 1) || (a.ss_ld & 1) || a.ss_ld < a.ss_n || a.k_real < 1 || a.k_real > a.k) return TF_EINVAL;
             if (a.half < 0 || 2 * a.half > a.R || a.max_pos < 1 || (a.half && (!a.cos || !a.sin))) return TF_EINVAL;
             if (a.kv_raw && (!a.kv_norm_w || !a.cache || !a.slot || a.ld_kv < a.C + a.R || a.c_real < 1 || a.c_real > a.C
                              || a.cache_rows < 1)) return TF_EINVAL;
@@ -299,7 +286,7 @@ extern "C" int tfl_gemm(const TflGemm* p, int dtype, int x_mode, int epi, void* 
             if (!a.out_t || !a.gate || a.ld_t < 8 || a.ld_gate < (int64_t)a.groups * a.n || (a.ld_t & 7) || (a.ld_gate & 3)) return TF_EINVAL;
             break;
         case TFL_EPI_RESIDUAL:
-            if (!a.out_f || a.groups != 1 || a.ld_f < a.n || (a.ld_f & 3)) return TF_EINVAL;
+            if (!a.out_f || a.groups != 1 || a.ld_f < a.n || (a.ld_f & 3) || (a.out_t && (a.ld_t < 8 || (a.ld_t & 7)))) return TF_EINVAL;
             break;
         case TFL_EPI_TOKEN:
             if (!a.out_t || !a.ids || !a.tok_table || a.groups != 1 || a.n_real < 1 || a.n_real > a.n || a.ld_tok < a.n_real
@@ -308,6 +295,5 @@ extern "C" int tfl_gemm(const TflGemm* p, int dtype, int x_mode, int epi, void* 
         default:
             return TF_EINVAL;
     }
-    return dtype == 0 ? dispatch_gemm<bf16>(a, x_mode, epi, (hipStream_t)stream)
-                      : dispatch_gemm<float>(a, x_mode, epi, (hipStream_t)stream);
+    return dtype == 0 ? dispatch_gemm<bf16>(a, epi, (hipStream_t)stream) : dispatch_gemm<float>(a, epi, (hipStream_t)stream);
 }

@@ -143,7 +143,6 @@ _lib = None
 # ---- libtriforce_latent.so (include/triforce_latent.h) ------------------------------------------------------------------
 TFL_PAGE = 64
 TFL_EPI = {n: i for i, n in enumerate(("f32", "in", "query", "latent", "gated", "residual", "token"))}
-TFL_X = {"t": 0, "f32": 1, "f32_norm": 2}
 
 
 class TflGemm(_c.Structure):
@@ -151,14 +150,14 @@ class TflGemm(_c.Structure):
     _fields_ = ([(n, _vp) for n in ("wp", "x", "norm_w", "ss_in", "out_t", "out_t2", "out_f", "ss_out", "gate", "tok_table", "ids",
                                     "pos", "cos", "sin", "kv_raw", "kv_norm_w", "cache", "slot")]
                 + [(n, _i64) for n in ("ld_x", "x_oct", "x_group", "ld_t", "t_oct", "ld_f", "ld_gate", "ld_tok", "ld_kv")]
-                + [(n, _i32) for n in ("rows", "n", "k", "groups", "n_real", "k_real", "n_raw", "ss_n", "ss_ld", "H", "N", "R", "C",
+                + [(n, _i32) for n in ("rows", "n", "k", "groups", "n_real", "k_real", "n_raw", "n_scaled", "ss_n", "ss_ld", "H", "N", "R", "C",
                                        "half", "c_real", "max_pos", "cache_rows", "vocab")]
                 + [("eps", _f32)])
 
 
 LATENT_SIGNATURES = {
     "tfl_abi_version": (_i32, []),
-    "tfl_gemm": (_i32, [_c.POINTER(TflGemm), _i32, _i32, _i32, _vp]),
+    "tfl_gemm": (_i32, [_c.POINTER(TflGemm), _i32, _i32, _vp]),
     "tfl_finish": (_i32, [_vp, _vp, _i32, _vp, _i32, _i64, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _i32, _i32, _i32, _f32, _i32, _vp]),
     "tfl_residual": (_i32, [_vp, _vp, _vp, _i64, _i32, _vp]),
     "tfl_token_gate": (_i32, [_vp, _i64, _vp, _i64, _vp, _i32, _vp, _i32, _i32, _i32, _i32, _vp]),

@@ -109,15 +109,15 @@ class LatentLayer:
     def decode(self, h, x, ids, side_table, batch, rope, cache_rows, eps):
         g = self.geom
         act = ol.empty_act(ids.numel(), self.w_out.k, h.dtype, h.device)
-        raw, ss = ol.input_projection(h, self.w_in, g.n_raw, act, g.H * g.V)
-        qn, q = ol.query_and_append(raw, ss, self.w_uq, g, self.q_norm, self.kv_norm, eps, rope, batch.pos, batch.slot, cache_rows)
+        raw, ss, xq = ol.input_projection(h, self.w_in, g.n_raw, self.q_norm, act, g.H * g.V)
+        qn, q = ol.query_and_append(xq, raw, ss, self.w_uq, g, self.kv_norm, eps, rope, batch.pos, batch.slot, cache_rows)
         ol.query_to_latent(qn, self.w_uk_t, q, g)
         o = ol.attn_decode(q, cache_rows, batch.table, batch.klen, g, self.scale, batch.max_len)
         ol.latent_to_value(o, self.w_uv, raw, g.gate_off, act, g)
-        ol.add_linear(act, self.w_out, x)
+        xt = ol.add_linear(act, self.w_out, x, want_copy=bool(self.side_dim))
         if not self.side_dim:
             return None
-        return ol.linear_f32(ol.token_gate_linear(x, self.side_gate, side_table, ids, self.side_dim), self.side_proj, self.width)
+        return ol.linear_f32(ol.token_gate_linear(xt, self.side_gate, side_table, ids, self.side_dim), self.side_proj, self.width)
 
     def prefill(self, h, x, ids, side_table, batch, rope, cache_rows, eps):
         g = self.geom

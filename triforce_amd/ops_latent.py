@@ -95,14 +95,14 @@ def _tail(x, k):
     return x[k // 8:] if x.dim() == 3 else x[:, k:]
 
 
-def _gemm(wt, x, x_mode, epi, rows, **kw):
+def _gemm(wt, x, epi, rows, **kw):
     a = hip.TflGemm()
     a.wp, a.x = wt.packed.data_ptr(), x.data_ptr()
     a.rows, a.n, a.k, a.groups = rows, wt.n, wt.k, wt.groups
     a.x_oct = a.t_oct = 8
     for name, v in kw.items():
         setattr(a, name, v.data_ptr() if isinstance(v, torch.Tensor) else v)
-    hip.check(hip.latent_lib().tfl_gemm(ctypes.byref(a), _CODE[wt.dtype], hip.TFL_X[x_mode], hip.TFL_EPI[epi], _stream()), "tfl_gemm " + epi)
+    hip.check(hip.latent_lib().tfl_gemm(ctypes.byref(a), _CODE[wt.dtype], hip.TFL_EPI[epi], _stream()), "tfl_gemm " + epi)
 
 
 def linear_f32(x, wt, n_real, out=None):
@@ -113,39 +113,43 @@ def linear_f32(x, wt, n_real, out=None):
     if out is None:
         out = torch.empty(rows, n_real, dtype=torch.float32, device=x.device)
     assert out.dtype == torch.float32 and out.shape[0] == rows and out.shape[1] >= n_real and out.stride(1) == 1
-    _gemm(wt, x, "t", "f32", rows, ld_x=ld, x_oct=octet, out_f=out, ld_f=out.stride(0), n_real=n_real)
+    _gemm(wt, x, "f32", rows, ld_x=ld, x_oct=octet, out_f=out, ld_f=out.stride(0), n_real=n_real)
     return out
 
 
-def input_projection(h, wt, n_raw, act, act_off):
+def input_projection(h, wt, n_raw, q_norm, act, act_off):
     """All projections of the layer's one norm (h, act: activation blocks).  Returns (raw fp32 [rows, n_raw], per-panel sums of
-    squares); gelu of the other outputs goes to the columns of act from act_off on."""
+    squares, the first len(q_norm) outputs times q_norm as an octet-major block); gelu of the outputs behind n_raw goes to the
+    columns of act from act_off on."""
     _need(h, act)
     rows, k, ld, octet = _lay(h)
     act_rows_, act_k, act_ld, act_oct = _lay(act)
     assert h.dtype == wt.dtype == act.dtype and k == wt.k and act_rows_ == rows and act_k >= act_off + wt.n - n_raw and act_off % 8 == 0
     raw = torch.empty(rows, n_raw, dtype=torch.float32, device=h.device)
     ss = torch.empty(rows, n_raw // 16, dtype=torch.float32, device=h.device)
+    _f32(q_norm)
+    xq = empty_act(rows, q_norm.numel(), wt.dtype, h.device)
     tail = _tail(act, act_off) if wt.n > n_raw else act
-    _gemm(wt, h, "t", "in", rows, ld_x=ld, x_oct=octet, out_f=raw, ld_f=n_raw, ss_out=ss, ss_ld=n_raw // 16, n_raw=n_raw,
-          out_t=tail, ld_t=act_ld, t_oct=act_oct)
-    return raw, ss
+    _gemm(wt, h, "in", rows, ld_x=ld, x_oct=octet, out_f=raw, ld_f=n_raw, ss_out=ss, ss_ld=n_raw // 16, n_raw=n_raw,
+          out_t=tail, ld_t=act_ld, t_oct=act_oct, out_t2=xq, norm_w=q_norm, n_scaled=q_norm.numel())
+    return raw, ss, xq
 
 
-def query_and_append(raw, ss, wt, g, q_norm, kv_norm, eps, rope, pos, slot, cache):
-    """Second stage of a decode step: raw's query latent normalised and up-projected (returned as unrotated [rows, H, N] and
-    [rows, H, C + R] with the rotated part filled in), raw's key latent normalised / rotated into the cache rows ``slot``.
-    g: LatentGeom."""
-    _need(raw, ss, cache, pos, slot)
+def query_and_append(xq, raw, ss, wt, g, kv_norm, eps, rope, pos, slot, cache):
+    """Second stage of a decode step: the weighted query latent xq up-projected and scaled by its norm (returned as unrotated
+    [rows, H, N] and [rows, H, C + R] with the rotated part filled in), raw's key latent normalised / rotated into the cache rows
+    ``slot``.  g: LatentGeom."""
+    _need(xq, raw, ss, cache, pos, slot)
     _i32(pos, slot)
-    _f32(raw, ss, q_norm, kv_norm)
-    rows = raw.shape[0]
+    _f32(raw, ss, kv_norm)
+    rows, k, ld, octet = _lay(xq)
+    assert k == g.Q and xq.dtype == wt.dtype and raw.shape[0] == rows
     assert wt.n == g.H * (g.N + g.R) and wt.k == g.Q and cache.dtype == wt.dtype and cache.shape[1] == g.C + g.R and cache.is_contiguous()
     assert pos.numel() == rows and slot.numel() == rows and raw.stride(0) == raw.shape[1] >= g.Q + g.C + g.R
     qn = torch.empty(rows, g.H, g.N, dtype=wt.dtype, device=raw.device)
     q = torch.empty(rows, g.H, g.C + g.R, dtype=wt.dtype, device=raw.device)
     kv = raw[:, g.Q:]
-    _gemm(wt, raw, "f32_norm", "query", rows, ld_x=raw.stride(0), norm_w=q_norm, ss_in=ss, ss_n=g.Q // 16, ss_ld=ss.shape[1],
+    _gemm(wt, xq, "query", rows, ld_x=ld, x_oct=octet, ss_in=ss, ss_n=g.Q // 16, ss_ld=ss.shape[1],
           k_real=g.q_real, eps=eps, out_t=q, out_t2=qn, pos=pos, cos=rope.cos, sin=rope.sin, half=rope.half, max_pos=rope.max_pos,
           H=g.H, N=g.N, R=g.R, C=g.C, c_real=g.c_real, kv_raw=kv, ld_kv=raw.stride(0), kv_norm_w=kv_norm, cache=cache,
           cache_rows=cache.shape[0], slot=slot)
@@ -157,7 +161,7 @@ def query_to_latent(qn, wt, q, g):
     _need(qn, q)
     rows = qn.shape[0]
     assert (wt.groups, wt.n, wt.k) == (g.H, g.C, g.N) and qn.dtype == q.dtype == wt.dtype
-    _gemm(wt, qn, "t", "latent", rows, ld_x=g.H * g.N, x_group=g.N, out_t=q, H=g.H, C=g.C, R=g.R)
+    _gemm(wt, qn, "latent", rows, ld_x=g.H * g.N, x_group=g.N, out_t=q, H=g.H, C=g.C, R=g.R)
     return q
 
 
@@ -167,26 +171,29 @@ def latent_to_value(ol, wt, raw, gate_off, act, g):
     rows, (act_rows_, act_k, act_ld, act_oct) = ol.shape[0], _lay(act)
     assert (wt.groups, wt.n, wt.k) == (g.H, g.V, g.C) and ol.dtype == act.dtype == wt.dtype and act_rows_ == rows and act_k >= g.H * g.V
     assert raw.shape[1] >= gate_off + g.H * g.V
-    _gemm(wt, ol, "t", "gated", rows, ld_x=g.H * g.C, x_group=g.C, gate=raw[:, gate_off:], ld_gate=raw.stride(0), out_t=act,
+    _gemm(wt, ol, "gated", rows, ld_x=g.H * g.C, x_group=g.C, gate=raw[:, gate_off:], ld_gate=raw.stride(0), out_t=act,
           ld_t=act_ld, t_oct=act_oct)
 
 
-def add_linear(act, wt, x):
-    """x (fp32) += act . W^T."""
+def add_linear(act, wt, x, want_copy=False):
+    """x (fp32) += act . W^T; returns the sum as an octet-major block of act's type when ``want_copy``."""
     _need(act, x)
     _f32(x)
     rows, k, ld, octet = _lay(act)
     assert act.dtype == wt.dtype and k == wt.k and x.shape == (rows, wt.n) and x.is_contiguous()
-    _gemm(wt, act, "t", "residual", rows, ld_x=ld, x_oct=octet, out_f=x, ld_f=x.stride(0))
+    xt = empty_act(rows, wt.n, wt.dtype, x.device) if want_copy else None
+    _gemm(wt, act, "residual", rows, ld_x=ld, x_oct=octet, out_f=x, ld_f=x.stride(0),
+          **(dict(out_t=xt, ld_t=8, t_oct=8 * rows) if want_copy else {}))
+    return xt
 
 
 def token_gate_linear(x, wt, table, ids, n_real):
-    """gelu(T(x) . W^T) * table[ids]: table is a column slice [vocab, n_real] of the token-side embedding."""
+    """gelu(x . W^T) * table[ids]: x an activation block, table a column slice [vocab, n_real] of the token-side embedding."""
     _need(x, table, ids)
-    _f32(x)
-    assert ids.dtype == torch.int64 and ids.numel() == x.shape[0] and table.dtype == wt.dtype and table.shape[1] == n_real
-    out = torch.empty(x.shape[0], wt.n, dtype=wt.dtype, device=x.device)
-    _gemm(wt, x, "f32", "token", x.shape[0], ld_x=x.stride(0), out_t=out, ld_t=wt.n, ids=ids, tok_table=table, ld_tok=table.stride(0),
+    rows, k, ld, octet = _lay(x)
+    assert ids.dtype == torch.int64 and ids.numel() == rows and k == wt.k and x.dtype == table.dtype == wt.dtype and table.shape[1] == n_real
+    out = torch.empty(rows, wt.n, dtype=wt.dtype, device=x.device)
+    _gemm(wt, x, "token", rows, ld_x=ld, x_oct=octet, out_t=out, ld_t=wt.n, ids=ids, tok_table=table, ld_tok=table.stride(0),
           vocab=table.shape[0], n_real=n_real)
     return out
 

@@ -1,7 +1,7 @@
 """Plain, slow restatement of the Befidra design (torch CPU): one function per mechanism, one sequence at a time, no cache.
 
-TEST INFRASTRUCTURE ONLY: the checker of tests/test_latent_*.py; the product (triforce_amd/) never imports it and it imports
-nothing from the product.  Everything runs in the dtype of the weights it is given (float32 or float64).
+TEST INFRASTRUCTURE ONLY: what tests/test_latent_cpu.py and tests/test_gpu_latent.py compare with; the product (triforce_amd/)
+never imports it and it imports nothing from the product.  Everything runs in the dtype of the weights it is given (float32 or float64).
 
 ``operand`` (everywhere): what happens to an activation right before a matrix product - nothing, or a rounding, which tells how
 far a product in a shorter format may move the result.
